@@ -19,7 +19,6 @@ import stat
 import subprocess
 import sys
 import tempfile
-import threading
 import time
 
 CSRC = os.path.dirname(os.path.abspath(__file__))
@@ -123,15 +122,6 @@ def build(force: bool = False, verbose: bool = True) -> str:
     started = time.time()
     if verbose:
         _say(f"compiling {len(names)} HIP sources for {OFFLOAD_ARCH} into {folder}")
-    stop = threading.Event()
-
-    def heartbeat() -> None:
-        while not stop.wait(20.0):
-            _say(f"still compiling ({time.time() - started:.0f} s)")
-
-    beat = threading.Thread(target=heartbeat, daemon=True)
-    if verbose:
-        beat.start()
 
     def compile_one(name: str) -> str:
         obj = os.path.join(folder, name[:-4] + ".o")
@@ -143,21 +133,18 @@ def build(force: bool = False, verbose: bool = True) -> str:
             _say(f"compiled {name} ({time.time() - started:.0f} s)")
         return obj
 
-    try:
-        workers = max(1, min(len(names), int(os.environ.get("MAX_JOBS", "0")) or (os.cpu_count() or 4), 16))
-        with concurrent.futures.ThreadPoolExecutor(max_workers=workers) as pool:
-            objects = list(pool.map(compile_one, names))
-        lib = os.path.join(folder, LIB_NAME)
-        tmp = lib + f".{os.getpid()}.tmp"
-        link = subprocess.run([hipcc, f"--offload-arch={OFFLOAD_ARCH}", "-shared", "-fPIC", *objects, "-o", tmp],
-                              capture_output=True, text=True)
-        if link.returncode != 0:
-            raise KernelBuildError(f"hipcc failed to link {LIB_NAME}:\n{link.stderr[-4000:]}")
-        os.replace(tmp, lib)
-        with open(os.path.join(folder, "digest.txt"), "w", encoding="utf-8") as handle:
-            handle.write(source_digest() + "\n")
-    finally:
-        stop.set()
+    workers = max(1, min(len(names), int(os.environ.get("MAX_JOBS", "0")) or (os.cpu_count() or 4), 16))
+    with concurrent.futures.ThreadPoolExecutor(max_workers=workers) as pool:
+        objects = list(pool.map(compile_one, names))
+    lib = os.path.join(folder, LIB_NAME)
+    tmp = lib + f".{os.getpid()}.tmp"
+    link = subprocess.run([hipcc, f"--offload-arch={OFFLOAD_ARCH}", "-shared", "-fPIC", *objects, "-o", tmp],
+                          capture_output=True, text=True)
+    if link.returncode != 0:
+        raise KernelBuildError(f"hipcc failed to link {LIB_NAME}:\n{link.stderr[-4000:]}")
+    os.replace(tmp, lib)
+    with open(os.path.join(folder, "digest.txt"), "w", encoding="utf-8") as handle:
+        handle.write(source_digest() + "\n")
     if verbose:
         _say(f"built {LIB_NAME} in {time.time() - started:.0f} s")
     return lib
