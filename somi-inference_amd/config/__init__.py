@@ -9,6 +9,8 @@ from .metitar import (MetitarConfig, MetitarDense, MetitarExperts, MetitarHGRN2,
                       RampedScaling)
 from .qwen2 import Qwen2Config
 from .rusolorn import RusolornAttention, RusolornConfig, RusolornDeltaRule, RusolornExperts, RusolornLayer
+from .tomopel import (TomopelAttention, TomopelConfig, TomopelDense, TomopelExperts, TomopelLayer, TomopelMamba2,
+                      TomopelMinGRU, TomopelParallel)
 from .registry import (Architecture, config_from_dict, register_architecture,
                        registered_architectures, resolve_architecture, unregister_architecture)
 
@@ -18,7 +20,8 @@ __all__ = [
     "GizilornLatentAttention", "GizilornLayer", "KamedraAttention", "KamedraConfig", "KamedraGLA", "KamedraLayer", "KeyReader",
     "MetitarConfig", "MetitarDense", "MetitarExperts", "MetitarHGRN2", "MetitarLatentAttention", "MetitarLayer", "RampedScaling",
     "ModelConfig", "Qwen2Config", "RotaryScaling", "RusolornAttention", "RusolornConfig", "RusolornDeltaRule",
-    "RusolornExperts", "RusolornLayer",
+    "RusolornExperts", "RusolornLayer", "TomopelAttention", "TomopelConfig", "TomopelDense", "TomopelExperts", "TomopelLayer",
+    "TomopelMamba2", "TomopelMinGRU", "TomopelParallel",
     "architecture_of", "config_from_dict", "normalize_dtype", "read_config_json",
     "register_architecture", "registered_architectures", "resolve_architecture",
     "unregister_architecture",

@@ -214,6 +214,37 @@ extern "C" int somi_xielu(const float* z, const float* pq, void* out, int out_dt
     return 0;
 }
 
+// The square of relu on float32 sums, rounded once.
+template <typename TO>
+__global__ void __launch_bounds__(256)
+squared_relu_kernel(const float* __restrict__ z, TO* __restrict__ out, int64_t count) {
+    const int64_t quads = count >> 2;
+    auto unit = [](float v) { v = fmaxf(v, 0.f); return v * v; };
+    for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < quads; i += (int64_t)gridDim.x * 256) {
+        const float4 v = reinterpret_cast<const float4*>(z)[i];
+        TO r[4] = {from_float<TO>(unit(v.x)), from_float<TO>(unit(v.y)), from_float<TO>(unit(v.z)), from_float<TO>(unit(v.w))};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) out[i * 4 + e] = r[e];
+    }
+    for (int64_t i = quads * 4 + (int64_t)blockIdx.x * 256 + threadIdx.x; i < count; i += (int64_t)gridDim.x * 256)
+        out[i] = from_float<TO>(unit(z[i]));
+}
+
+extern "C" int somi_squared_relu(const float* z, void* out, int out_dtype, int64_t count, hipStream_t stream) {
+    SOMI_REQUIRE(count >= 0, "squared_relu: bad sizes");
+    SOMI_REQUIRE(((uintptr_t)z & 15) == 0, "squared_relu: rows must start at a multiple of 16 bytes");
+    if (count == 0) return 0;
+    const int grid = (int)(ceil_div64(count, 1024) < 65536 ? ceil_div64(count, 1024) : 65536);
+    if (out_dtype == SOMI_F32)
+        hipLaunchKernelGGL(squared_relu_kernel<float>, dim3(grid), dim3(256), 0, stream, z, (float*)out, count);
+    else if (out_dtype == SOMI_BF16)
+        hipLaunchKernelGGL(squared_relu_kernel<bf16>, dim3(grid), dim3(256), 0, stream, z, (bf16*)out, count);
+    else
+        return somi_fail("squared_relu: unknown dtype %d", out_dtype);
+    SOMI_LAUNCH_CHECK("squared_relu");
+    return 0;
+}
+
 // A sigmoid gate on rows: out = x * sigmoid(g) element by element; g: float32 sums of the gate's product, rows
 // g_stride apart; x and out: [n, width] of one type.
 template <typename T>

@@ -15,6 +15,7 @@
 //                   four consecutive keys of one channel with one 8-byte load)
 // The wavefronts of a workgroup are merged through LDS; with several splits the workgroup writes
 // (max, sum, unnormalised output) to a workspace and a second kernel merges the splits in split order.
+#include "attention_bias.h"
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -250,13 +251,15 @@ __device__ __forceinline__ float lanes4_sum(float v) {
 // captured step of requests at 4,096 to 8,192 tokens allows) is one split, with four workgroups of head size 128 still
 // fitting a compute unit's LDS (38 KB each).
 #define DECODE_LDS_PAGES 768
-template <int DT>
+// BIAS: a distance bias is added to the scores (attention_bias.h); the rows of the workgroup's heads are in LDS where
+// they fit, in the units of the unscaled scores.
+template <int DT, bool BIAS>
 __global__ void __launch_bounds__(256)
 attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc,
                             const bf16* __restrict__ vc, const int* __restrict__ block_table, int max_blocks,
                             const int* __restrict__ token_list, const int* __restrict__ token_entry,
                             const int* __restrict__ positions, int nq, int nkv, int page_size, int window,
-                            float scale, int split_len, int num_splits, bf16* __restrict__ out,
+                            float scale, int split_len, int num_splits, DistanceBias bias, bf16* __restrict__ out,
                             float* __restrict__ part_acc, float* __restrict__ part_ml) {
     constexpr int D = DT * 16;
     constexpr int QK_STEPS = (DT + 1) / 2;
@@ -268,6 +271,7 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
     __shared__ __attribute__((aligned(16))) bf16 ks[2][32 * KROW];
     __shared__ __attribute__((aligned(16))) bf16 vs[2][D * VROW];
     __shared__ int pages[DECODE_LDS_PAGES];
+    extern __shared__ float bias_s[];                        // BIAS, in_lds: [min(G, 16)][bias.length]
 
     // the key/value heads of a token are neighbours in the grid: they start together and walk the same pages at the
     // same pace, so that the 4 KB pieces of a page that they read (one per head, next to each other) are asked for
@@ -313,6 +317,16 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
         const int page_lo = (begin & ~31) >> shift, page_last = end >> shift;
         const int page_count = ((end | 31) >> shift) - page_lo + 1;
         for (int i = tid; i < page_count; i += 256) pages[i] = table[min(page_lo + i, page_last)];
+        // the bias of this split's keys: only a split that reaches the token's nearest keys has any
+        const float inv_scale = 1.0f / scale;
+        const int bias_rows = G < 16 ? G : 16;
+        const int bias_row = r < bias_rows ? r : bias_rows - 1;
+        if (BIAS && bias.in_lds && p - end < bias.length) {
+            for (int i = tid; i < bias_rows * bias.length; i += 256) {
+                const int hl = hb * 16 + i / bias.length;
+                bias_s[i] = bias.table[(int64_t)(kvh * G + (hl < G ? hl : G - 1)) * bias.length + i % bias.length] * inv_scale;
+            }
+        }
         __syncthreads();
         auto page_of = [&](int pos) -> int64_t { return pages[(pos >> shift) - page_lo]; };
         const int64_t page_stride = (int64_t)nkv * page_size * D;      // elements from one page to the next
@@ -377,6 +391,16 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
                     u.half4[1] = short4_t{0, 0, 0, 0};
                     s[half] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u.wide, qf[QK_STEPS - 1], s[half], 0, 0, 0);
                 }
+            }
+            if (BIAS && p - (j0 + 31) < bias.length) {
+#pragma unroll
+                for (int half = 0; half < 2; ++half)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        const int n = bias_index(p - (j0 + half * 16 + g * 4 + i), bias.length);
+                        s[half][i] += bias.in_lds ? bias_s[bias_row * bias.length + n]
+                                                  : bias.table[(int64_t)head * bias.length + n] * inv_scale;
+                    }
             }
             // s[half][i] = S[key j0 + 16 half + 4 g + i][head r], still unscaled; keys outside the split are
             // masked (only the first and last step of a split can hold any)
@@ -525,18 +549,29 @@ template <int DT>
 static int launch_decode(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                          int max_blocks, const int* token_list, const int* token_entry, const int* positions,
                          int n_list, int nq, int nkv, int page_size, int window, float scale, int split_len,
-                         int num_splits, void* out, float* part_acc, float* part_ml, hipStream_t stream) {
+                         int num_splits, DistanceBias bias, void* out, float* part_acc, float* part_ml,
+                         hipStream_t stream) {
     const int waves = DT <= 8 ? 4 : 2;
     const int G = nq / nkv, HB = (G + 15) / 16;
     const size_t smem = (size_t)(waves * DT * 256 + waves * 32) * sizeof(float);
     const bool pow2_pages = (page_size & (page_size - 1)) == 0;
-    if (DT >= 2 && DT <= 8 && pow2_pages && n_list <= 65535 &&
-        split_len / page_size + 2 + 8 <= DECODE_LDS_PAGES)                                        // + a tile's overhang
+    const bool staged = DT >= 2 && DT <= 8 && pow2_pages && n_list <= 65535 &&
+                        split_len / page_size + 2 + 8 <= DECODE_LDS_PAGES;                        // + a tile's overhang
+    if (bias.length > 0) {
+        SOMI_REQUIRE(staged, "attention_decode: a distance bias comes with head sizes 32 to 128, pages of a power of two "
+                     "keys and splits whose pages fit LDS (head size %d, pages of %d, splits of %d)", DT * 16, page_size, split_len);
+        const int floats = (G < 16 ? G : 16) * bias.length;
+        bias.in_lds = floats <= BIAS_LDS_FLOATS;
+        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), true>), dim3(nkv * HB, n_list, num_splits),
+                           dim3(256), bias.in_lds ? floats * sizeof(float) : 0, stream, (const bf16*)q, q_stride,
+                           (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, token_list, token_entry, positions,
+                           nq, nkv, page_size, window, scale, split_len, num_splits, bias, (bf16*)out, part_acc, part_ml);
+    } else if (staged)
         // head sizes 32..128: keys and values staged through LDS (two tiles fit)
-        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2)>), dim3(nkv * HB, n_list, num_splits),
+        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), false>), dim3(nkv * HB, n_list, num_splits),
                            dim3(256), 0, stream, (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table,
                            max_blocks, token_list, token_entry, positions, nq, nkv, page_size, window, scale, split_len,
-                           num_splits, (bf16*)out, part_acc, part_ml);
+                           num_splits, bias, (bf16*)out, part_acc, part_ml);
     else
         hipLaunchKernelGGL((attention_decode_kernel<DT>), dim3(n_list, nkv * HB, num_splits), dim3(waves * 64), smem,
                            stream, (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks,
@@ -556,12 +591,13 @@ static int launch_decode(const void* q, int64_t q_stride, const void* kc, const 
 // page_size a multiple of 4.  k_cache [pages, nkv, page_size, D], v_cache [pages, nkv, D, page_size].
 // With num_splits > 1, part_acc holds n_list * nq * num_splits * D floats and part_ml
 // n_list * nq * num_splits * 2 floats; split_len is a multiple of 16 and split_len * num_splits covers every
-// listed token's position.
+// listed token's position.  bias_table: [nq, bias_length] float32 or null (attention_bias.h).
 extern "C" int somi_attention_decode(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                                      const int* block_table, int max_blocks, const int* token_list,
                                      const int* token_entry, const int* positions, int n_list, int nq, int nkv, int D,
-                                     int page_size, int window, float scale, int split_len, int num_splits, void* out,
-                                     float* part_acc, float* part_ml, hipStream_t stream) {
+                                     int page_size, int window, float scale, int split_len, int num_splits,
+                                     const float* bias_table, int bias_length, void* out, float* part_acc,
+                                     float* part_ml, hipStream_t stream) {
     SOMI_REQUIRE(n_list >= 0 && nq > 0 && nkv > 0 && max_blocks > 0, "attention_decode: bad sizes");
     SOMI_REQUIRE(nq % nkv == 0, "attention_decode: num_q_heads (%d) must be divisible by num_kv_heads (%d)", nq, nkv);
     SOMI_REQUIRE(D % 16 == 0 && D >= 16 && D <= 256, "attention_decode: head_dim %d must be a multiple of 16 up to 256", D);
@@ -574,11 +610,14 @@ extern "C" int somi_attention_decode(const void* q, int64_t q_stride, const void
                  (uintptr_t)v_cache % 8 == 0, "attention_decode: q, k and v must be 16-byte aligned");
     const int G = nq / nkv, HB = (G + 15) / 16;
     SOMI_REQUIRE(nkv * HB <= 65535, "attention_decode: too many heads");
+    SOMI_REQUIRE(bias_length >= 0 && (bias_length == 0 || (bias_table != nullptr && scale > 0.f)),
+                 "attention_decode: a distance bias needs its table and a scale above 0");
     if (n_list == 0) return 0;
+    const DistanceBias bias{bias_table, bias_length, 0};
 #define SOMI_DECODE(DT)                                                                                              \
     case DT:                                                                                                         \
         return launch_decode<DT>(q, q_stride, k_cache, v_cache, block_table, max_blocks, token_list, token_entry,    \
-                                 positions, n_list, nq, nkv, page_size, window, scale, split_len, num_splits, out,   \
+                                 positions, n_list, nq, nkv, page_size, window, scale, split_len, num_splits, bias, out, \
                                  part_acc, part_ml, stream)
     switch (D / 16) {
         SOMI_DECODE(1); SOMI_DECODE(2); SOMI_DECODE(3); SOMI_DECODE(4); SOMI_DECODE(5); SOMI_DECODE(6);

@@ -17,6 +17,7 @@
 //                                            inside a page, so a lane reads 2 x 4 consecutive keys of a channel
 // Every key tile is used for all QB query blocks from registers.  Key tiles are aligned to absolute
 // positions (multiples of 32), so a query's arithmetic does not depend on how the prompt was cut.
+#include "attention_bias.h"
 #include "common.h"
 #include "attention_prefill_tile.h"
 
@@ -253,12 +254,14 @@ static int prefill_key_split_below(int units) { return 7 * units / 2; }      // 
 // KS = 2: twice the wavefronts; each query block is owned by KS of them, which take the 32-key tiles in turn
 // (tile index modulo KS, by absolute position) and join their sums, maxima and outputs through LDS at the
 // end.  The longest workgroup, which sets the time of a short prompt, has half as many steps to walk.
-template <int DT, int QB, int KS>
+// BIAS: a distance bias is added to the scores (attention_bias.h); its head's row is in LDS behind the page list where it
+// fits, in the units of the unscaled scores.
+template <int DT, int QB, int KS, bool BIAS>
 __global__ void __launch_bounds__(256 * KS, 2 * KS)     // the second figure: wavefronts per SIMD to leave room for
 attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc,
                              const bf16* __restrict__ vc, const int* __restrict__ block_table, int max_blocks,
                              const int* __restrict__ entry_start, const int* __restrict__ entry_first_pos, const int* __restrict__ entry_len, int nq,
-                             int nkv, int page_size, int window, float scale_log2, bf16* __restrict__ out) {
+                             int nkv, int page_size, int window, float scale_log2, DistanceBias bias, int bias_at, bf16* __restrict__ out) {
     constexpr int D = DT * 16;
     constexpr int QK_STEPS = (DT + 1) / 2;
     constexpr int QW = QB * 16, WAVES = 4, QG = WAVES * QW;             // 64 or 128 queries per workgroup
@@ -307,6 +310,11 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
     const int page_lo = (lo & ~(STEP - 1)) >> shift, page_last = wg_last >> shift;
     const int page_count = (((wg_last | (STEP - 1)) >> shift) - page_lo) + 1;
     for (int i = tid; i < page_count; i += THREADS) pages[i] = table[min(page_lo + i, page_last)];
+    float* bias_s = reinterpret_cast<float*>(pages + bias_at);
+    const float* bias_row = bias.table + (int64_t)h * bias.length;
+    const float bias_unit = 1.44269504088896341f / scale_log2;          // the scores stay unscaled until the weights
+    if (BIAS && bias.in_lds)
+        for (int i = tid; i < bias.length; i += THREADS) bias_s[i] = bias_row[i] * bias_unit;
     __syncthreads();
     auto page_of = [&](int pos) -> int64_t { return pages[(pos >> shift) - page_lo]; };
     auto page_offset = [&](int pos) { return pos & (page_size - 1); };
@@ -428,6 +436,17 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
                     for (int c = 0; c < QK_STEPS; ++c)
                         s[qb][half] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[half][c], qf[qb][c], s[qb][half], 0, 0, 0);
                 }
+            if (BIAS && pos0 + q0 - (j0 + 31) < bias.length) {
+#pragma unroll
+                for (int qb = 0; qb < QB; ++qb)
+#pragma unroll
+                    for (int half = 0; half < 2; ++half)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) {
+                            const int n = bias_index(pcol[qb] - (j0 + half * 16 + g * 4 + i), bias.length);
+                            s[qb][half][i] += bias.in_lds ? bias_s[n] : bias_row[n] * bias_unit;
+                        }
+            }
             // scores stay unscaled; keys a query must not see are masked, which only steps that reach past the
             // wavefront's first query (or a window's lower edge) can hold
             if (window > 0 || j0 + 31 > pos0 + q0) {
@@ -588,36 +607,36 @@ template <int DT>
 static int launch_prefill_lds(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                               int max_blocks, const int* entry_start, const int* entry_first_pos, const int* entry_len, int n_entries,
                               int max_entry_len, int max_context, int shape, int nq, int nkv, int page_size,
-                              int window, float scale, void* out, hipStream_t stream) {
-    const size_t page_list = (size_t)prefill_page_entries(max_blocks, page_size, window) * sizeof(int);
+                              int window, float scale, DistanceBias bias, void* out, hipStream_t stream) {
+    const int bias_at = prefill_page_entries(max_blocks, page_size, window);
+    size_t page_list = (size_t)bias_at * sizeof(int);             // dynamic LDS: the page list, then the bias if it fits
+    bias.in_lds = bias.length > 0 && bias.length <= BIAS_LDS_FLOATS &&
+                  (int)page_list + bias.length * 4 + prefill_lds_static(DT * 16, 1) <= PREFILL_LDS_TOTAL;
+    if (bias.in_lds) page_list += bias.length * sizeof(float);
     const bool split_fits = (int)page_list + prefill_lds_static(DT * 16, 2) <= PREFILL_LDS_TOTAL;
     if (shape == PREFILL_SHAPE_AUTO)
         shape = prefill_lds_choice(n_entries, max_entry_len, max_context, nq, window, split_fits, somi_units());
     const bool wide = shape == PREFILL_SHAPE_WIDE;
     const dim3 grid(nq, n_entries, ceil_div(max_entry_len, wide ? 128 : 64));
+#define PREFILL_LDS_LAUNCH(QB, KS, BIAS)                                                                                    \
+    do {                                                                                                                    \
+        if (page_list > 16 * 1024)                       /* with the tiles beyond the default limit of LDS */               \
+            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, QB, KS, BIAS>,                          \
+                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)page_list);                          \
+        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, QB, KS, BIAS>), grid, dim3(256 * KS), page_list, stream,       \
+                           (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start, \
+                           entry_first_pos, entry_len, nq, nkv, page_size, window, scale * 1.44269504088896341f, bias,      \
+                           bias_at, (bf16*)out);                                                                            \
+    } while (0)
     if (wide) {
-        if (page_list > 16 * 1024)                       // with the tiles beyond the default limit of LDS
-            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, 2, 1>,
-                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)page_list);
-        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, 2, 1>), grid, dim3(256), page_list, stream, (const bf16*)q,
-                           q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start,
-                           entry_first_pos, entry_len, nq, nkv, page_size, window, scale * 1.44269504088896341f, (bf16*)out);
+        if (bias.length > 0) PREFILL_LDS_LAUNCH(2, 1, true); else PREFILL_LDS_LAUNCH(2, 1, false);
     } else if (shape == PREFILL_SHAPE_SPLIT && split_fits) {
         // few workgroups with many tiles each: the keys of a query block are split over two wavefronts
-        if (page_list > 16 * 1024)
-            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, 1, 2>,
-                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)page_list);
-        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, 1, 2>), grid, dim3(512), page_list, stream, (const bf16*)q,
-                           q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start,
-                           entry_first_pos, entry_len, nq, nkv, page_size, window, scale * 1.44269504088896341f, (bf16*)out);
+        if (bias.length > 0) PREFILL_LDS_LAUNCH(1, 2, true); else PREFILL_LDS_LAUNCH(1, 2, false);
     } else {
-        if (page_list > 16 * 1024)
-            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, 1, 1>,
-                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)page_list);
-        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, 1, 1>), grid, dim3(256), page_list, stream, (const bf16*)q,
-                           q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start,
-                           entry_first_pos, entry_len, nq, nkv, page_size, window, scale * 1.44269504088896341f, (bf16*)out);
+        if (bias.length > 0) PREFILL_LDS_LAUNCH(1, 1, true); else PREFILL_LDS_LAUNCH(1, 1, false);
     }
+#undef PREFILL_LDS_LAUNCH
     SOMI_LAUNCH_CHECK("attention_prefill_lds");
     return 0;
 }
@@ -644,12 +663,12 @@ static int launch_prefill(const void* q, int64_t q_stride, const void* kc, const
 // up to 256; page_size a multiple of 4.  k_cache [pages, nkv, page_size, D], v_cache [pages, nkv, D, page_size];
 // out: [n_tokens, nq * D].  max_context: the longest context a portion ends at (a hint for the launch shape; 0: unknown).
 // shape: 0 lets the launcher choose; 1..3 ask for a launch shape of the 16 x 16 LDS kernel, 4 and 5 for one of the
-// 32 x 32 tile kernel (PREFILL_SHAPE_*).
+// 32 x 32 tile kernel (PREFILL_SHAPE_*).  bias_table: [nq, bias_length] float32 or null (attention_bias.h).
 extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                                       const int* block_table, int max_blocks, const int* entry_start,
                                       const int* entry_first_pos, const int* entry_len, int n_entries, int max_entry_len, int max_context,
                                       int shape, int nq, int nkv, int D, int page_size, int window, float scale,
-                                      void* out, hipStream_t stream) {
+                                      const float* bias_table, int bias_length, void* out, hipStream_t stream) {
     SOMI_REQUIRE(n_entries >= 0 && max_entry_len >= 0 && nq > 0 && nkv > 0 && max_blocks > 0,
                  "attention_prefill: bad sizes");
     SOMI_REQUIRE(nq % nkv == 0, "attention_prefill: num_q_heads (%d) must be divisible by num_kv_heads (%d)", nq, nkv);
@@ -663,7 +682,10 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
     SOMI_REQUIRE((uintptr_t)q % 16 == 0 && (q_stride * 2) % 16 == 0 && (uintptr_t)k_cache % 16 == 0 &&
                  (uintptr_t)v_cache % 8 == 0 && (uintptr_t)out % 8 == 0,
                  "attention_prefill: q, k, v and out must be 16-byte aligned");
+    SOMI_REQUIRE(bias_length >= 0 && (bias_length == 0 || (bias_table != nullptr && scale > 0.f)),
+                 "attention_prefill: a distance bias needs its table and a scale above 0");
     if (n_entries == 0 || max_entry_len == 0) return 0;
+    const DistanceBias bias{bias_table, bias_length, 0};
     // head sizes 64 and 128 over pages of 8 keys or more: the 32 x 32 tile kernel
     const bool tile_ok = somi_prefill_tile_applies(D, page_size, max_blocks, window) && (uintptr_t)v_cache % 16 == 0;
     if (shape >= PREFILL_SHAPE_TILE)
@@ -673,7 +695,7 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
         const int64_t groups = (int64_t)ceil_div(max_entry_len, 256) * n_entries * nq;
         const bool wide = shape == PREFILL_SHAPE_AUTO ? groups >= prefill_tile_wide_groups(somi_units()) : shape == PREFILL_SHAPE_TILE_WIDE;
         return somi_prefill_tile(q, q_stride, k_cache, v_cache, block_table, max_blocks, entry_start, entry_first_pos, entry_len,
-                                 n_entries, max_entry_len, wide, nq, nkv, D, page_size, window, scale, out, stream);
+                                 n_entries, max_entry_len, wide, nq, nkv, D, page_size, window, scale, bias, out, stream);
     }
 #define SOMI_PREFILL(DT, QB)                                                                                       \
     case DT:                                                                                                       \
@@ -688,12 +710,15 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
                                          scale, out, stream);                                                      \
         return launch_prefill_lds<DT>(q, q_stride, k_cache, v_cache, block_table, max_blocks, entry_start,         \
                                       entry_first_pos, entry_len, n_entries, max_entry_len, max_context, shape, nq, nkv,      \
-                                      page_size, window, scale, out, stream)
+                                      page_size, window, scale, bias, out, stream)
     // head sizes 32..128 stage keys and values through LDS; the others (LDS would not hold two tiles, or a
     // tile is smaller than the workgroup's loads) keep them in registers per wavefront, and so do page sizes
     // that are no power of two and block tables too wide for the LDS copy of a request's pages
     const bool lds_ok = (page_size & (page_size - 1)) == 0 &&
                         prefill_page_entries(max_blocks, page_size, window) * 4 + prefill_lds_static(D, 1) <= PREFILL_LDS_TOTAL;
+    SOMI_REQUIRE(bias_length == 0 || (lds_ok && D >= 32 && D <= 128),
+                 "attention_prefill: a distance bias comes with head sizes 32 to 128 and pages of a power of two keys whose "
+                 "list fits LDS (head size %d, pages of %d)", D, page_size);
     switch (D / 16) {
         SOMI_PREFILL(1, 4); SOMI_PREFILL_LDS(2); SOMI_PREFILL_LDS(3); SOMI_PREFILL_LDS(4); SOMI_PREFILL_LDS(5);
         SOMI_PREFILL_LDS(6); SOMI_PREFILL_LDS(7); SOMI_PREFILL_LDS(8); SOMI_PREFILL(9, 2); SOMI_PREFILL(10, 2);
@@ -716,4 +741,12 @@ extern "C" int somi_attention_prefill_choice(int n_entries, int max_entry_len, i
         return groups >= prefill_tile_wide_groups(units) ? PREFILL_SHAPE_TILE_WIDE : PREFILL_SHAPE_TILE;
     }
     return prefill_lds_choice(n_entries, max_entry_len, max_context, nq, window, split_fits != 0, units);
+}
+
+// Whether the matrix-core kernels take a distance bias at these sizes: both the prompts' and the decoded tokens' kernel
+// must be one of those that stage keys through LDS.
+extern "C" int somi_attention_bias_supported(int D, int page_size, int max_blocks) {
+    if (D % 16 != 0 || D < 32 || D > 128 || page_size < 4 || (page_size & (page_size - 1)) != 0) return 0;
+    return somi_prefill_tile_applies(D, page_size, max_blocks, 0) ||
+           prefill_page_entries(max_blocks, page_size, 0) * 4 + prefill_lds_static(D, 1) <= PREFILL_LDS_TOTAL;
 }

@@ -63,12 +63,15 @@ __device__ __forceinline__ float tile_pair_max(float v) {
 }
 
 // D: head size (64 or 128).  QBLK query blocks of 32 per workgroup, KS key splits; QBLK * KS wavefronts.
-template <int D, int QBLK, int KS>
+// BIAS: a distance bias is added to the scores (attention_bias.h); its head's row is in LDS behind the page list where it
+// fits, in the units of the score product.
+template <int D, int QBLK, int KS, bool BIAS>
 __global__ void __launch_bounds__(QBLK * KS * 64, 2)
 prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
                     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ entry_start,
                     const int* __restrict__ entry_first_pos, const int* __restrict__ entry_len, int nq, int nkv,
-                    int page_size, int window, float scale_pow2, float scale_rest, bf16* __restrict__ out) {
+                    int page_size, int window, float scale_pow2, float scale_rest, DistanceBias bias, int bias_at,
+                    bf16* __restrict__ out) {
     constexpr int THREADS = QBLK * KS * 64;
     constexpr int CH = D / 8;                    // 16-byte pieces of a key row
     constexpr int KROW = D * 2;                  // bytes
@@ -103,6 +106,11 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
     const int page_lo = j_begin >> shift, page_last = wg_last >> shift;
     const int page_count = (((wg_last | (STEP - 1)) >> shift) - page_lo) + 1;
     for (int i = tid; i < page_count; i += THREADS) pages[i] = table[min(page_lo + i, page_last)];
+    float* bias_s = reinterpret_cast<float*>(pages + bias_at);
+    const float* bias_row = bias.table + (int64_t)h * bias.length;
+    const float bias_unit = 1.44269504088896341f / scale_rest;
+    if (BIAS && bias.in_lds)
+        for (int i = tid; i < bias.length; i += THREADS) bias_s[i] = bias_row[i] * bias_unit;
     __syncthreads();
     const int64_t page_bytes = (int64_t)nkv * page_size * D * 2;       // bytes from one page to the next
     const char* k_head = reinterpret_cast<const char*>(kc) + (int64_t)kvh * page_size * D * 2;
@@ -243,6 +251,16 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
                 for (int t = 0; t < 2; ++t)
                     vf[b][t] = *(const TILE_LDS bf16x8*)(vaddr[t] + (ST + b * 2048));
             TILE_FENCE();
+            if (BIAS && w_first - (j0 + 31) < bias.length) {
+                const int n0 = p_rel - j0;                     // register r: n0 - (16 (r / 8) + r % 8) keys back
+                if (bias.in_lds) {
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) sc[r] += bias_s[bias_index(n0 - (16 * (r >> 3) + (r & 7)), bias.length)];
+                } else {
+#pragma unroll
+                    for (int r = 0; r < 16; ++r) sc[r] += bias_row[bias_index(n0 - (16 * (r >> 3) + (r & 7)), bias.length)] * bias_unit;
+                }
+            }
             if (j0 + 31 > w_first) {
                 const int lim = p_rel - j0;
 #pragma unroll
@@ -367,17 +385,28 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
         }
 }
 
-template <int D, int QBLK, int KS>
+// Entries of a workgroup's page list: its visible pages and a step's overhang.
+static int tile_page_entries(int qblk, int max_blocks, int page_size, int window) {
+    const int entries = max_blocks + 64 / page_size + 2;
+    return window > 0 ? min(entries, (window + qblk * 32 + 128) / page_size + 4) : entries;
+}
+
+template <int D, int QBLK, int KS, bool BIAS>
 static int launch_tile(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table, int max_blocks,
                        const int* entry_start, const int* entry_first_pos, const int* entry_len, int n_entries,
-                       int max_entry_len, int nq, int nkv, int page_size, int window, float scale, void* out,
-                       hipStream_t stream) {
-    const int lds = somi_prefill_tile_lds(D, QBLK, KS, max_blocks, page_size, window);
+                       int max_entry_len, int nq, int nkv, int page_size, int window, float scale, DistanceBias bias,
+                       void* out, hipStream_t stream) {
+    // dynamic LDS: the stages and the page list, then (BIAS) the head's row if it fits
+    const int bias_at = tile_page_entries(QBLK, max_blocks, page_size, window);
+    const int with_bias = 2 * KS * (32 * D * 2 + D * 64) + (bias_at + bias.length) * 4;
+    int lds = somi_prefill_tile_lds(D, QBLK, KS, max_blocks, page_size, window);
+    bias.in_lds = BIAS && bias.length <= BIAS_LDS_FLOATS && with_bias <= SOMI_PREFILL_TILE_LDS_MAX;
+    if (bias.in_lds) lds = max(lds, with_bias);
     static int lds_allowed[64];                  // per device: the largest dynamic LDS this kernel has been allowed so far
     int device = 0;
     if (hipGetDevice(&device) != hipSuccess || device < 0 || device >= 64) return somi_fail("attention_prefill_tile: hipGetDevice failed");
     if (lds > lds_allowed[device]) {
-        const hipError_t err = hipFuncSetAttribute((const void*)prefill_tile_kernel<D, QBLK, KS>,
+        const hipError_t err = hipFuncSetAttribute((const void*)prefill_tile_kernel<D, QBLK, KS, BIAS>,
                                                    hipFuncAttributeMaxDynamicSharedMemorySize, lds);
         if (err != hipSuccess) return somi_fail("attention_prefill_tile: %d bytes of LDS refused: %s", lds, hipGetErrorString(err));
         lds_allowed[device] = lds;
@@ -387,9 +416,9 @@ static int launch_tile(const void* q, int64_t q_stride, const void* kc, const vo
     int exponent = 0;
     const float rest = 2.f * frexpf(scale * 1.44269504088896341f, &exponent);
     const float pow2 = ldexpf(1.f, exponent - 1);
-    hipLaunchKernelGGL((prefill_tile_kernel<D, QBLK, KS>), grid, dim3(QBLK * KS * 64), lds, stream, (const bf16*)q, q_stride,
+    hipLaunchKernelGGL((prefill_tile_kernel<D, QBLK, KS, BIAS>), grid, dim3(QBLK * KS * 64), lds, stream, (const bf16*)q, q_stride,
                        (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start, entry_first_pos, entry_len,
-                       nq, nkv, page_size, window, pow2, rest, (bf16*)out);
+                       nq, nkv, page_size, window, pow2, rest, bias, bias_at, (bf16*)out);
     SOMI_LAUNCH_CHECK("attention_prefill_tile");
     return 0;
 }
@@ -397,9 +426,7 @@ static int launch_tile(const void* q, int64_t q_stride, const void* kc, const vo
 // Dynamic LDS of a launch: two stages of tiles, the request's visible pages, and what the key splits hand over.
 int somi_prefill_tile_lds(int D, int qblk, int ks, int max_blocks, int page_size, int window) {
     const int tile = 32 * D * 2 + D * 64;
-    int entries = max_blocks + 64 / page_size + 2;
-    if (window > 0) entries = min(entries, (window + qblk * 32 + 128) / page_size + 4);
-    int lds = 2 * ks * tile + entries * 4;
+    int lds = 2 * ks * tile + tile_page_entries(qblk, max_blocks, page_size, window) * 4;
     if (ks == 2) lds = max(lds, qblk * (D / 32 * 16 + 2) * 256);
     return lds;
 }
@@ -416,14 +443,21 @@ bool somi_prefill_tile_applies(int D, int page_size, int max_blocks, int window)
 int somi_prefill_tile(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                       int max_blocks, const int* entry_start, const int* entry_first_pos, const int* entry_len,
                       int n_entries, int max_entry_len, bool wide, int nq, int nkv, int D, int page_size, int window,
-                      float scale, void* out, hipStream_t stream) {
-#define SOMI_TILE(DD, QB, KS_)                                                                                          \
-    return launch_tile<DD, QB, KS_>(q, q_stride, kc, vc, block_table, max_blocks, entry_start, entry_first_pos, entry_len, \
-                                    n_entries, max_entry_len, nq, nkv, page_size, window, scale, out, stream)
+                      float scale, DistanceBias bias, void* out, hipStream_t stream) {
+#define SOMI_TILE_AS(DD, QB, KS_, BIAS)                                                                                 \
+    return launch_tile<DD, QB, KS_, BIAS>(q, q_stride, kc, vc, block_table, max_blocks, entry_start, entry_first_pos,    \
+                                          entry_len, n_entries, max_entry_len, nq, nkv, page_size, window, scale, bias, \
+                                          out, stream)
+#define SOMI_TILE(DD, QB, KS_)                                \
+    do {                                                      \
+        if (bias.length > 0) SOMI_TILE_AS(DD, QB, KS_, true); \
+        SOMI_TILE_AS(DD, QB, KS_, false);                     \
+    } while (0)
     if (D == 128 && wide) SOMI_TILE(128, 8, 1);
     if (D == 128) SOMI_TILE(128, 4, 2);
     if (D == 64 && wide) SOMI_TILE(64, 8, 1);
     if (D == 64) SOMI_TILE(64, 4, 2);
 #undef SOMI_TILE
+#undef SOMI_TILE_AS
     return somi_fail("attention_prefill_tile: head size %d is not taken", D);
 }

@@ -9,42 +9,12 @@
 // Before that q, k and v pass a short causal convolution over time per channel (taps[c, last] weighs the current
 // token, zeros before a sequence's start) and SiLU; the last taps - 1 inputs of a request are state as well.
 //
-// Four kernels: `conv` (convolution and SiLU) and `unit` (unit norms, beta, decay), which together leave everything
-// the recurrence reads in float32; `conv_state` (the convolution's inputs that the next step needs); `scan` (the
-// recurrence).
+// The convolution with SiLU (short_conv.hip) and the kernel `unit` (unit norms, beta, decay) together leave everything the
+// recurrence reads in float32; `scan` is the recurrence.
 #include "common.h"
+#include "short_conv.h"
 
-#define DELTA_MAX_TAPS 9        // conv_state keeps taps - 1 <= 8 values a channel in registers
-
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
-// The convolution: a thread per (token, channel).  x: the token's row [q (G dim) | k (G dim) | v (H vdim) | ...] as
-// projected; taps: [C, taps] float32 for the C = 2 G dim + H vdim channels in that order; conv_state: [slots,
-// taps - 1, C] float32, the inputs before the entry's first token, oldest first.
-template <typename T>
-__global__ void __launch_bounds__(256)
-delta_conv_kernel(const T* __restrict__ x, int64_t row_stride, const float* __restrict__ taps_w, int taps,
-                  const float* __restrict__ conv_state, const int* __restrict__ token_entry,
-                  const int* __restrict__ entry_start, const int* __restrict__ state_slots, int C,
-                  float* __restrict__ qkv_out /*[N, C]*/) {
-    const int64_t t = blockIdx.x;
-    const int c = blockIdx.y * 256 + threadIdx.x;
-    if (c >= C) return;
-    const int e = token_entry[t];
-    const int i = (int)t - entry_start[e];
-    const int64_t slot = state_slots[e];
-    float acc = 0.f;
-#pragma unroll
-    for (int d = 0; d < DELTA_MAX_TAPS; ++d) {
-        if (d >= taps) break;
-        const float w = taps_w[c * taps + taps - 1 - d];
-        const float xv = i - d >= 0 ? to_float(x[(t - d) * row_stride + c])
-                                    : conv_state[(slot * (taps - 1) + (taps - 1 + i - d)) * C + c];
-        acc += w * xv;
-    }
-    qkv_out[t * C + c] = silu_f(acc);
-}
 
 // One workgroup per token, after the convolution: unit vectors per q and k head (2 G heads of dim channels, q heads
 // first; q also times dim^-1/2), and beta and the decay from ab: [N, 2 H] float32, the projections behind beta (first
@@ -69,31 +39,6 @@ delta_unit_kernel(const float* __restrict__ ab, const float* __restrict__ a_log,
         ss = wave_sum(ss);
         const float inv = (head < G ? q_scale : 1.0f) / sqrtf(ss + 1e-6f);
         for (int d = lane; d < dim; d += 64) p[d] *= inv;
-    }
-}
-
-// After `conv`: the last taps - 1 inputs of every entry's request, from the step's rows and, where the entry is
-// shorter than that, from what the state held.  A thread reads all of a channel's values before it writes any.
-template <typename T>
-__global__ void __launch_bounds__(256)
-delta_conv_state_kernel(const T* __restrict__ x, int64_t row_stride, int taps, float* __restrict__ conv_state,
-                        const int* __restrict__ entry_start, const int* __restrict__ state_slots, int C) {
-    const int e = blockIdx.x;
-    const int c = blockIdx.y * 256 + threadIdx.x;
-    if (c >= C) return;
-    const int start = entry_start[e], len = entry_start[e + 1] - start;
-    float* st = conv_state + (int64_t)state_slots[e] * (taps - 1) * C;
-    float vals[DELTA_MAX_TAPS - 1];
-#pragma unroll
-    for (int s = 0; s < DELTA_MAX_TAPS - 1; ++s) {
-        if (s >= taps - 1) break;
-        const int j = len - (taps - 1) + s;          // index among the entry's tokens; negative: before the entry
-        vals[s] = j >= 0 ? to_float(x[(int64_t)(start + j) * row_stride + c]) : st[(taps - 1 + j) * C + c];
-    }
-#pragma unroll
-    for (int s = 0; s < DELTA_MAX_TAPS - 1; ++s) {
-        if (s >= taps - 1) break;
-        st[s * C + c] = vals[s];
     }
 }
 
@@ -226,32 +171,17 @@ delta_scan_kernel(const float* __restrict__ qkv /*[N, C]*/, const float* __restr
 extern "C" int somi_delta_prepare(const void* x, int dtype, int64_t row_stride, const float* ab, const float* taps_w,
                                   int taps, float* conv_state, const int* token_entry, const int* entry_start,
                                   const int* state_slots, const float* a_log, const float* dt_bias, int n_tokens,
-                                  int n_entries, int groups, int heads, int dim, int vdim, float* qkv_out, float* beta,
-                                  float* decay, hipStream_t stream) {
+                                  int n_entries, int max_entry_len, int groups, int heads, int dim, int vdim,
+                                  float* qkv_out, float* beta, float* decay, hipStream_t stream) {
     SOMI_REQUIRE(n_tokens >= 0 && n_entries >= 0 && groups > 0 && heads > 0 && heads % groups == 0 && dim > 0 && vdim > 0,
                  "delta_prepare: bad sizes");
-    SOMI_REQUIRE(taps >= 1 && taps <= DELTA_MAX_TAPS, "delta_prepare: %d taps, at most %d are supported", taps, DELTA_MAX_TAPS);
-    SOMI_REQUIRE(ceil_div(2 * groups * dim + heads * vdim, 256) <= 65535, "delta_prepare: too many channels");
     const int C = 2 * groups * dim + heads * vdim;
     SOMI_REQUIRE(row_stride >= C, "delta_prepare: rows too narrow");
     if (n_tokens == 0) return 0;
-    const dim3 cgrid(n_entries, ceil_div(C, 256));
-    const dim3 tgrid(n_tokens, ceil_div(C, 256));
-    if (dtype == SOMI_F32) {
-        hipLaunchKernelGGL(delta_conv_kernel<float>, tgrid, dim3(256), 0, stream, (const float*)x, row_stride, taps_w, taps,
-                           conv_state, token_entry, entry_start, state_slots, C, qkv_out);
-        if (taps > 1)
-            hipLaunchKernelGGL(delta_conv_state_kernel<float>, cgrid, dim3(256), 0, stream, (const float*)x, row_stride, taps,
-                               conv_state, entry_start, state_slots, C);
-    } else if (dtype == SOMI_BF16) {
-        hipLaunchKernelGGL(delta_conv_kernel<bf16>, tgrid, dim3(256), 0, stream, (const bf16*)x, row_stride, taps_w, taps,
-                           conv_state, token_entry, entry_start, state_slots, C, qkv_out);
-        if (taps > 1)
-            hipLaunchKernelGGL(delta_conv_state_kernel<bf16>, cgrid, dim3(256), 0, stream, (const bf16*)x, row_stride, taps,
-                               conv_state, entry_start, state_slots, C);
-    } else {
-        return somi_fail("delta_prepare: unknown dtype %d", dtype);
-    }
+    // x: the token's row [q (groups dim) | k (groups dim) | v (heads vdim) | ...] as projected
+    if (somi_short_conv(x, dtype, row_stride, taps_w, nullptr, taps, conv_state, token_entry, entry_start, state_slots,
+                        n_tokens, n_entries, max_entry_len, C, qkv_out, stream))
+        return 1;
     hipLaunchKernelGGL(delta_unit_kernel, dim3(n_tokens), dim3(256), 0, stream, ab, a_log, dt_bias, groups, heads, dim, vdim,
                        qkv_out, beta, decay);
     SOMI_LAUNCH_CHECK("delta_prepare");

@@ -4,11 +4,13 @@
 //   route      z = W_r h (float32), s = softmax(z) or, element by element, sigmoid(z); experts come in `groups` equal
 //              runs of neighbours, a run scores as its best expert and only the `keep` best runs stay; of their experts
 //              the `top` with the largest s are chosen, weighted by s over the chosen scores' sum (+ 1e-20) or by s as
-//              it is.  Ties go to the lower index.
+//              it is.  With a `correction` per expert the choice looks at s + correction, the weights at s alone.  Ties go
+//              to the lower index.
 //   align      the N * top pairs sorted by expert: order[], the experts' offsets and a list of row tiles
 //              (expert, first sorted row, rows) that the products' grids walk.
 //   gate_up    act[p, :] = glu(W_gate[e] h_t, W_up[e] h_t) for the sorted pair p = (t, e); where the pair's weight is to
 //              multiply the expert's input, glu(w_pair W_gate[e] h_t, w_pair W_up[e] h_t): the float32 sums are scaled
+//   up         the same for experts without a gate: act[p, :] = relu(W_up[e] h_t)^2
 //   down       y[pair, :] = w_pair * (W_down[e] act[p, :]) (or without the weight), float32, at the pair's own place
 //              t * top + j
 //   combine    out[t, :] = sum_j y[t * top + j, :] (+ shared[t, :]), float32, in the order of j
@@ -20,6 +22,15 @@
 #define MOE_MAX_EXPERTS 256
 #define MOE_MAX_TOP 32
 #define MOE_TILE_ROWS 16
+
+// What an experts' product does: `down` over sorted rows, or over rows gathered by token, ending in the gated unit or in
+// the squared relu.
+enum MoeMode { MOE_DOWN = 0, MOE_GATED = 1, MOE_SQUARED_RELU = 2 };
+
+__device__ __forceinline__ float squared_relu(float v) {
+    v = fmaxf(v, 0.f);
+    return v * v;
+}
 
 __device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
     g = fminf(g, limit);
@@ -127,11 +138,12 @@ __device__ __forceinline__ void wave_best(float& value, int& index) {
 template <typename T>
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __restrict__ router,
-                 const float* __restrict__ logits, int width, int experts,
+                 const float* __restrict__ logits, const float* __restrict__ correction, int width, int experts,
                  int top, int groups, int keep, int sigmoid_scores, int normalize, int* __restrict__ chosen,
                  float* __restrict__ weight) {
     constexpr int PER_LANE = MOE_MAX_EXPERTS / 64;
     __shared__ float score[MOE_MAX_EXPERTS];
+    __shared__ float pure[MOE_MAX_EXPERTS];         // the scores before the correction: what the weights are made of
     __shared__ int taken[MOE_MAX_EXPERTS];          // per run: kept or not
     __shared__ float pick_score[MOE_MAX_TOP];
     __shared__ int pick_index[MOE_MAX_TOP];
@@ -171,7 +183,11 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
 #pragma unroll
     for (int j = 0; j < PER_LANE; ++j) {
         s[j] /= total;
-        if (lane + 64 * j < experts) score[lane + 64 * j] = s[j];
+        if (lane + 64 * j < experts) {
+            pure[lane + 64 * j] = s[j];
+            if (correction != nullptr) s[j] += correction[lane + 64 * j];
+            score[lane + 64 * j] = s[j];
+        }
     }
     for (int g = lane; g < groups; g += 64) taken[g] = keep >= groups ? 1 : 0;
     __syncthreads();
@@ -182,14 +198,14 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
 #pragma unroll
         for (int j = 0; j < PER_LANE; ++j) {
             const int g = lane + 64 * j;
-            run[j] = -1.f;
+            run[j] = -INFINITY;
             if (g < groups) {
                 run[j] = score[g * per];
                 for (int i = 1; i < per; ++i) run[j] = fmaxf(run[j], score[g * per + i]);
             }
         }
         for (int round = 0; round < keep; ++round) {
-            float best = -1.f;
+            float best = -INFINITY;
             int best_run = 1 << 30;
 #pragma unroll
             for (int j = 0; j < PER_LANE; ++j)
@@ -202,7 +218,7 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
 #pragma unroll
             for (int j = 0; j < PER_LANE; ++j)
                 if (lane + 64 * j == best_run) {
-                    run[j] = -1.f;
+                    run[j] = -INFINITY;
                     taken[best_run] = 1;
                 }
         }
@@ -211,11 +227,11 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
 #pragma unroll
     for (int j = 0; j < PER_LANE; ++j) {
         const int e = lane + 64 * j;
-        if (e >= experts || !taken[e / per]) s[j] = -1.f;  // out of the choice
+        if (e >= experts || !taken[e / per]) s[j] = -INFINITY;  // out of the choice
     }
     float sum = 0.f;
     for (int pick = 0; pick < top; ++pick) {
-        float best = -1.f;
+        float best = -INFINITY;
         int best_expert = 1 << 30;
 #pragma unroll
         for (int j = 0; j < PER_LANE; ++j)
@@ -226,11 +242,11 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
         wave_best(best, best_expert);
         if (best_expert >= experts) {                      // scores that compare with nothing: any expert, weight as it comes
             best_expert = 0;
-            best = score[0];
         }
 #pragma unroll
         for (int j = 0; j < PER_LANE; ++j)
-            if (lane + 64 * j == best_expert) s[j] = -1.f;
+            if (lane + 64 * j == best_expert) s[j] = -INFINITY;
+        best = pure[best_expert];
         if (lane == 0) {
             pick_score[pick] = best;
             pick_index[pick] = best_expert;
@@ -244,8 +260,8 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
     }
 }
 
-extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, const float* router, float* logits,
-                              int n_tokens, int width, int experts, int top, int groups, int keep, int sigmoid_scores,
+extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, const float* router, const float* correction,
+                              float* logits, int n_tokens, int width, int experts, int top, int groups, int keep, int sigmoid_scores,
                               int normalize, int* chosen, float* weight, hipStream_t stream) {
     SOMI_REQUIRE(n_tokens >= 0 && width > 0 && experts > 0 && experts <= MOE_MAX_EXPERTS, "moe_route: %d experts, 1 to %d are supported",
                  experts, MOE_MAX_EXPERTS);
@@ -272,10 +288,10 @@ extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, cons
     }
     if (dtype == SOMI_F32)
         hipLaunchKernelGGL(moe_route_kernel<float>, dim3(n_tokens), dim3(64), 0, stream, (const float*)x, row_stride, router,
-                           tiled ? logits : nullptr, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
+                           tiled ? logits : nullptr, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
     else
         hipLaunchKernelGGL(moe_route_kernel<bf16>, dim3(n_tokens), dim3(64), 0, stream, (const bf16*)x, row_stride, router,
-                           tiled ? logits : nullptr, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
+                           tiled ? logits : nullptr, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
     SOMI_LAUNCH_CHECK("moe_route");
     return 0;
 }
@@ -330,15 +346,17 @@ extern "C" int somi_moe_align(const int* chosen, int pairs, int experts, int til
 
 // The experts' products over the sorted rows, plain multiply-adds with float32 sums: a workgroup owns one row tile
 // (MOE_TILE_ROWS sorted rows of one expert) and 64 output columns, K goes through LDS 32 at a time.
-//   GATED: rows are gathered from x by token (pair / top); W: [experts, 2 F, K] (gate rows, then up rows); the end
+//   gated: rows are gathered from x by token (pair / top); W: [experts, 2 F, K] (gate rows, then up rows); the end
 //          applies the gated unit and writes act[sorted row, F] in T.
-//   else : rows are act's sorted rows; W: [experts, N, K]; the end multiplies by the pair's weight and writes
+//   squared relu: the same with W: [experts, F, K] and relu(.)^2 at the end.
+//   down : rows are act's sorted rows; W: [experts, N, K]; the end multiplies by the pair's weight and writes
 //          y[pair, N] in float32.
-template <typename T, bool GATED>
+template <typename T, int MODE>
 __global__ void __launch_bounds__(256)
 moe_product_kernel(const T* __restrict__ a, int64_t a_stride, const T* __restrict__ w, const int* __restrict__ tiles,
                    const int* __restrict__ order, const float* __restrict__ pair_weight, int top, int n_out, int K,
                    float limit, float alpha, float shift, void* __restrict__ out_) {
+    constexpr bool GATED = MODE == MOE_GATED, GATHER = MODE != MOE_DOWN;
     __shared__ float As[MOE_TILE_ROWS][33];
     __shared__ float Ws[64][33];
     __shared__ float Us[GATED ? 64 : 1][33];
@@ -358,7 +376,7 @@ moe_product_kernel(const T* __restrict__ a, int64_t a_stride, const T* __restric
             const int rr = i >> 5, kk = i & 31;
             float v = 0.f;
             if (rr < rows && k0 + kk < K) {
-                const int64_t src = GATED ? pair_of[rr] / top : first + rr;
+                const int64_t src = GATHER ? pair_of[rr] / top : first + rr;
                 v = to_float(a[src * a_stride + k0 + kk]);
             }
             As[rr][kk] = v;
@@ -390,13 +408,15 @@ moe_product_kernel(const T* __restrict__ a, int64_t a_stride, const T* __restric
         const float pw = pair_weight != nullptr ? pair_weight[pair] : 1.0f;
         if (GATED) {
             ((T*)out_)[(int64_t)(first + r) * n_out + c] = from_float<T>(clamped_glu(pw * acc[j], pw * acu[j], limit, alpha, shift));
+        } else if (MODE == MOE_SQUARED_RELU) {
+            ((T*)out_)[(int64_t)(first + r) * n_out + c] = from_float<T>(squared_relu(pw * acc[j]));
         } else {
             ((float*)out_)[(int64_t)pair * n_out + c] = pw * acc[j];
         }
     }
 }
 
-extern "C" int somi_moe_product(const void* a, int64_t a_stride, const void* w, int dtype, int gated, const int* tiles,
+extern "C" int somi_moe_product(const void* a, int64_t a_stride, const void* w, int dtype, int mode, const int* tiles,
                                 int max_tiles, const int* order, const float* pair_weight, int top, int n_out, int K,
                                 float limit, float alpha, float shift, void* out, hipStream_t stream) {
     SOMI_REQUIRE(max_tiles >= 0 && n_out > 0 && K > 0 && top > 0 && a_stride >= K, "moe_product: bad sizes");
@@ -406,10 +426,11 @@ extern "C" int somi_moe_product(const void* a, int64_t a_stride, const void* w, 
 #define SOMI_MOE(T, G)                                                                                                   \
     hipLaunchKernelGGL((moe_product_kernel<T, G>), grid, dim3(256), 0, stream, (const T*)a, a_stride, (const T*)w, tiles, order, \
                        pair_weight, top, n_out, K, limit, alpha, shift, out)
+    SOMI_REQUIRE(mode == MOE_DOWN || mode == MOE_GATED || mode == MOE_SQUARED_RELU, "moe_product: unknown mode %d", mode);
     if (dtype == SOMI_F32) {
-        if (gated) SOMI_MOE(float, true); else SOMI_MOE(float, false);
+        if (mode == MOE_GATED) SOMI_MOE(float, MOE_GATED); else if (mode == MOE_DOWN) SOMI_MOE(float, MOE_DOWN); else SOMI_MOE(float, MOE_SQUARED_RELU);
     } else if (dtype == SOMI_BF16) {
-        if (gated) SOMI_MOE(bf16, true); else SOMI_MOE(bf16, false);
+        if (mode == MOE_GATED) SOMI_MOE(bf16, MOE_GATED); else if (mode == MOE_DOWN) SOMI_MOE(bf16, MOE_DOWN); else SOMI_MOE(bf16, MOE_SQUARED_RELU);
     } else {
         return somi_fail("moe_product: unknown dtype %d", dtype);
     }
@@ -431,12 +452,13 @@ typedef __attribute__((ext_vector_type(4))) float moe_f32x4;
 // FRAGS: row fragments of a tile (4: up to 64 rows; 1: up to 16 rows, for steps of a few tokens, where a tile is an
 // expert's one or two rows and the time is the weights' way from memory).  KS: K steps of 32 whose fragments are asked
 // for together, a round ahead (1 with four row fragments; 4 with one, so that a lane has twenty loads in flight).
-template <bool GATED, int FRAGS, int KS>
+template <int MODE, int FRAGS, int KS>
 __global__ void __launch_bounds__(256)
 moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16* __restrict__ w,
                         const int* __restrict__ tiles, const int* __restrict__ order,
                         const float* __restrict__ pair_weight, int top, int n_out, int K, float limit, float alpha,
                         float shift, void* __restrict__ out_) {
+    constexpr bool GATED = MODE == MOE_GATED, GATHER = MODE != MOE_DOWN;
     const int expert = tiles[blockIdx.x * 3];
     if (expert < 0) return;
     const int first = tiles[blockIdx.x * 3 + 1], rows = tiles[blockIdx.x * 3 + 2];
@@ -453,7 +475,7 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
     for (int f = 0; f < FRAGS; ++f) {
         const int row = f * 16 + r;
         alive[f] = row < rows;
-        const int64_t src = alive[f] ? (GATED ? (int64_t)(order[first + row] / top) : (int64_t)(first + row)) : 0;
+        const int64_t src = alive[f] ? (GATHER ? (int64_t)(order[first + row] / top) : (int64_t)(first + row)) : 0;
         arow[f] = a + src * a_stride + g * 8;
     }
     const bf16* brow[4];
@@ -527,7 +549,9 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
 #pragma unroll
                 for (int c = 0; c < 4; ++c) {
                     const int col = col0 + c * 16 + r;
-                    if (col < n_out) ((float*)out_)[(int64_t)pair * n_out + col] = pw * acc[f][c][i];
+                    if (col >= n_out) continue;
+                    if (MODE == MOE_SQUARED_RELU) ((bf16*)out_)[(int64_t)(first + row) * n_out + col] = (bf16)squared_relu(pw * acc[f][c][i]);
+                    else ((float*)out_)[(int64_t)pair * n_out + col] = pw * acc[f][c][i];
                 }
             }
         }
@@ -545,12 +569,13 @@ typedef __attribute__((ext_vector_type(16))) float moe_f32x16;
 #define MOE_TILE_BK 64
 #define MOE_TILE_ROW_BYTES (MOE_TILE_BK * 2 + 16)
 
-template <bool GATED>
+template <int MODE>
 __global__ void __launch_bounds__(256)
 moe_product_tile_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16* __restrict__ w,
                         const int* __restrict__ tiles, const int* __restrict__ order,
                         const float* __restrict__ pair_weight, int top, int n_out, int K, float limit, float alpha,
                         float shift, void* __restrict__ out_) {
+    constexpr bool GATED = MODE == MOE_GATED, GATHER = MODE != MOE_DOWN;
     __shared__ __attribute__((aligned(16))) char lds_a[2][128 * MOE_TILE_ROW_BYTES];
     __shared__ __attribute__((aligned(16))) char lds_b[2][128 * MOE_TILE_ROW_BYTES];
     const int expert = tiles[blockIdx.x * 3];
@@ -572,7 +597,7 @@ moe_product_tile_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
         const int p = tid + 256 * j, row = p >> 3, piece = p & 7;
         soff[j] = row * MOE_TILE_ROW_BYTES + piece * 16;
         alive[j] = row < rows;
-        const int64_t src = alive[j] ? (GATED ? (int64_t)(order[first + row] / top) : (int64_t)(first + row)) : 0;
+        const int64_t src = alive[j] ? (GATHER ? (int64_t)(order[first + row] / top) : (int64_t)(first + row)) : 0;
         arow[j] = a + src * a_stride + piece * 8;
         // LDS row of the matrix: wavefront column wn' = row / 64, its fragment f = (row / 32) % 2, column c = row % 32
         const int wq = row >> 6, f = (row >> 5) & 1, c = row & 31;
@@ -655,13 +680,16 @@ moe_product_tile_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
 #pragma unroll
                     for (int j = 0; j < 2; ++j) {
                         const int col = col_base + wn * 64 + j * 32 + frow;
-                        if (col < n_out) ((float*)out_)[(int64_t)pair * n_out + col] = pw * acc[i][j][4 * g + e];
+                        if (col >= n_out) continue;
+                        const float v = pw * acc[i][j][4 * g + e];
+                        if (MODE == MOE_SQUARED_RELU) ((bf16*)out_)[(int64_t)(first + row) * n_out + col] = (bf16)squared_relu(v);
+                        else ((float*)out_)[(int64_t)pair * n_out + col] = v;
                     }
                 }
             }
 }
 
-extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void* w, int gated, const int* tiles,
+extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void* w, int mode, const int* tiles,
                                      int max_tiles, int tile_rows, const int* order, const float* pair_weight, int top,
                                      int n_out, int K, float limit, float alpha, float shift, void* out,
                                      hipStream_t stream) {
@@ -670,31 +698,25 @@ extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void
     SOMI_REQUIRE(max_tiles >= 0 && n_out > 0 && K > 0 && top > 0 && a_stride >= K, "moe_product_mfma: bad sizes");
     SOMI_REQUIRE(K % 8 == 0 && a_stride % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0,
                  "moe_product_mfma: K of %d or rows that are not aligned to 16 bytes", K);
+    SOMI_REQUIRE(mode == MOE_DOWN || mode == MOE_GATED || mode == MOE_SQUARED_RELU, "moe_product_mfma: unknown mode %d", mode);
     if (max_tiles == 0) return 0;
-    const dim3 grid(max_tiles, ceil_div(n_out, gated ? 128 : 256));
+    const int wide = tile_rows == MOE_BIG_ROWS ? 1 : 2;              // columns of a workgroup: 64 or 128 gated, else twice that
+    const dim3 grid(max_tiles, ceil_div(n_out, (mode == MOE_GATED ? 64 : 128) * wide));
     SOMI_REQUIRE(grid.y <= 65535, "moe_product_mfma: too many columns");
-    if (tile_rows == MOE_BIG_ROWS) {
-        const dim3 tgrid(max_tiles, ceil_div(n_out, gated ? 64 : 128));
-        SOMI_REQUIRE(tgrid.y <= 65535, "moe_product_mfma: too many columns");
-        if (gated)
-            hipLaunchKernelGGL(moe_product_tile_kernel<true>, tgrid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                               (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
-        else
-            hipLaunchKernelGGL(moe_product_tile_kernel<false>, tgrid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                               (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
-    } else if (tile_rows == 16) {
-        if (gated)
-            hipLaunchKernelGGL((moe_product_mfma_kernel<true, 1, 4>), grid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                               (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
-        else
-            hipLaunchKernelGGL((moe_product_mfma_kernel<false, 1, 4>), grid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                               (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
-    } else if (gated)
-        hipLaunchKernelGGL((moe_product_mfma_kernel<true, MOE_MFMA_FRAGS, 1>), grid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                           (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
-    else
-        hipLaunchKernelGGL((moe_product_mfma_kernel<false, MOE_MFMA_FRAGS, 1>), grid, dim3(256), 0, stream, (const bf16*)a, a_stride,
-                           (const bf16*)w, tiles, order, pair_weight, top, n_out, K, limit, alpha, shift, out);
+#define MOE_LAUNCH(...)                                                                                                   \
+    hipLaunchKernelGGL((__VA_ARGS__), grid, dim3(256), 0, stream, (const bf16*)a, a_stride, (const bf16*)w, tiles, order, \
+                       pair_weight, top, n_out, K, limit, alpha, shift, out)
+#define MOE_BY_ROWS(MODE)                                                                             \
+    do {                                                                                              \
+        if (tile_rows == MOE_BIG_ROWS) MOE_LAUNCH(moe_product_tile_kernel<MODE>);                     \
+        else if (tile_rows == 16) MOE_LAUNCH(moe_product_mfma_kernel<MODE, 1, 4>);                    \
+        else MOE_LAUNCH(moe_product_mfma_kernel<MODE, MOE_MFMA_FRAGS, 1>);                            \
+    } while (0)
+    if (mode == MOE_GATED) MOE_BY_ROWS(MOE_GATED);
+    else if (mode == MOE_DOWN) MOE_BY_ROWS(MOE_DOWN);
+    else MOE_BY_ROWS(MOE_SQUARED_RELU);
+#undef MOE_BY_ROWS
+#undef MOE_LAUNCH
     SOMI_LAUNCH_CHECK("moe_product_mfma");
     return 0;
 }

@@ -207,12 +207,24 @@ def rope_kv_store(qkv: torch.Tensor, positions: torch.Tensor, slots: torch.Tenso
                                         head_dim, _ptr(k_cache), _ptr(v_cache), page_size, _stream()))
 
 
+def _bias_arguments(bias: torch.Tensor | None, heads: int) -> tuple[ctypes.c_void_p, int]:
+    """A distance bias as the kernels take it: [heads, length] float32 added to the scaled score of the key n positions
+    back, relative to what far keys get (the last entry is 0 and stands for every key farther back)."""
+    if bias is None:
+        return _ptr(None), 0
+    _need(bias, "distance bias", torch.float32)
+    if bias.dim() != 2 or bias.shape[0] != heads or bias.shape[1] < 1:
+        raise KernelError(f"distance bias: expected [{heads}, length], got {tuple(bias.shape)}")
+    return _ptr(bias), bias.shape[1]
+
+
 def paged_attention_plain(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
                           block_table: torch.Tensor, token_entry: torch.Tensor, positions: torch.Tensor,
-                          nq: int, window: int, scale: float) -> torch.Tensor:
+                          nq: int, window: int, scale: float, bias: torch.Tensor | None = None) -> torch.Tensor:
     """Causal attention of every token over its request's cached keys (plain float32 kernel).
 
-    q: a tensor whose row t holds the nq query heads of token t first (row stride q_stride elements).
+    q: a tensor whose row t holds the nq query heads of token t first (row stride q_stride elements).  ``bias``: a
+    distance bias, see :func:`_bias_arguments`.
     """
     _need(q, "q")
     n = q.shape[0]
@@ -230,14 +242,15 @@ def paged_attention_plain(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor,
     _check(library().somi_paged_attention_plain(
         _ptr(q), dtype_code(q.dtype), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table),
         block_table.shape[1], _ptr(token_entry), _ptr(positions), n, nq, nkv, head_dim, page_size, window,
-        ctypes.c_float(scale), _ptr(out), _stream()))
+        ctypes.c_float(scale), *_bias_arguments(bias, nq), _ptr(out), _stream()))
     return out
 
 
 def attention_decode(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
                      block_table: torch.Tensor, token_entry: torch.Tensor, positions: torch.Tensor,
                      nq: int, window: int, scale: float, split_len: int, num_splits: int,
-                     out: torch.Tensor, token_list: torch.Tensor | None = None) -> None:
+                     out: torch.Tensor, token_list: torch.Tensor | None = None,
+                     bias: torch.Tensor | None = None) -> None:
     """MFMA attention of the listed tokens (all when ``token_list`` is None) over their pages, written
     into ``out`` ([N, nq * D] bfloat16).  The keys of a request are cut into ``num_splits`` ranges of
     ``split_len`` positions that run in parallel and are merged afterwards."""
@@ -265,13 +278,15 @@ def attention_decode(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_ca
     _check(library().somi_attention_decode(
         _ptr(q), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
         _ptr(token_list), _ptr(token_entry), _ptr(positions), n_list, nq, nkv, head_dim, page_size, window,
-        ctypes.c_float(scale), split_len, num_splits, _ptr(out), _ptr(part_acc), _ptr(part_ml), _stream()))
+        ctypes.c_float(scale), split_len, num_splits, *_bias_arguments(bias, nq), _ptr(out), _ptr(part_acc), _ptr(part_ml),
+        _stream()))
 
 
 def attention_prefill(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
                       block_table: torch.Tensor, entry_start: torch.Tensor, entry_first_position: torch.Tensor,
                       max_entry_len: int, nq: int, window: int, scale: float, out: torch.Tensor,
-                      max_context: int = 0, shape: int = 0, entry_len: torch.Tensor | None = None) -> None:
+                      max_context: int = 0, shape: int = 0, entry_len: torch.Tensor | None = None,
+                      bias: torch.Tensor | None = None) -> None:
     """MFMA causal attention of every token of every portion over its request's pages, into ``out``
     ([N, nq * D] bfloat16).  entry_start: [E + 1] int32 offsets of the portions in the flat batch;
     entry_first_position: [E] int32.  ``max_context``: the longest context a portion ends at, a hint for the
@@ -302,7 +317,7 @@ def attention_prefill(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_c
     _check(library().somi_attention_prefill(
         _ptr(q), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
         _ptr(entry_start), _ptr(entry_first_position), _ptr(entry_len), entries, max_entry_len, max(0, int(max_context)), int(shape), nq, nkv,
-        head_dim, page_size, window, ctypes.c_float(scale), _ptr(out), _stream()))
+        head_dim, page_size, window, ctypes.c_float(scale), *_bias_arguments(bias, nq), _ptr(out), _stream()))
 
 
 def silu_mul(gate_up: torch.Tensor, block: int = 0) -> torch.Tensor:
@@ -1049,7 +1064,37 @@ def qk_norm_store(rows: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tenso
 
 
 # ------------------------------------------------------------------------------------------ the gated delta rule
-DELTA_MAX_TAPS = 9
+SHORT_CONV_MAX_TAPS = 9
+
+
+def conv_silu(rows: torch.Tensor, taps: torch.Tensor, bias: torch.Tensor | None, conv_state: torch.Tensor, step) -> torch.Tensor:
+    """silu of a causal convolution over time per channel (+ bias) -> [N, C] float32.  rows: [N, C], possibly columns of
+    wider rows; taps: [C, taps] float32, the last on the current token; conv_state: [slots, max(taps - 1, 1), C] float32, a
+    request's last inputs, read and then advanced by the step's entries."""
+    if not isinstance(rows, torch.Tensor) or not rows.is_cuda or rows.dim() != 2 or rows.stride(1) != 1:
+        raise KernelError("conv_silu: the rows must be a matrix on the GPU with contiguous rows")
+    n, channels = rows.shape
+    _need(taps, "convolution taps", torch.float32)
+    if taps.dim() != 2 or taps.shape[0] != channels or not 1 <= taps.shape[1] <= SHORT_CONV_MAX_TAPS:
+        raise KernelError(f"conv_silu: taps {tuple(taps.shape)} != [{channels}, 1..{SHORT_CONV_MAX_TAPS}]")
+    width = taps.shape[1]
+    if bias is not None:
+        _need(bias, "convolution bias", torch.float32, (channels,))
+    _need(conv_state, "convolution state", torch.float32)
+    if tuple(conv_state.shape[1:]) != (max(width - 1, 1), channels):
+        raise KernelError(f"conv_silu: state {tuple(conv_state.shape)} != [slots, {max(width - 1, 1)}, {channels}]")
+    entries = step.state_slots.numel()
+    _need(step.token_entry, "token entries", torch.int32, (n,))
+    _need(step.entry_start, "entry offsets", torch.int32, (entries + 1,))
+    out = torch.empty((n, channels), dtype=torch.float32, device=rows.device)
+    _check(library().somi_conv_silu(_ptr(rows), dtype_code(rows.dtype), ctypes.c_int64(rows.stride(0)), _ptr(taps), _ptr(bias),
+                                    width, _ptr(conv_state), _ptr(step.token_entry), _ptr(step.entry_start),
+                                    _ptr(step.state_slots), n, entries, int(step.max_entry_len), channels, _ptr(out),
+                                    _stream()))
+    return out
+
+
+DELTA_MAX_TAPS = SHORT_CONV_MAX_TAPS
 
 
 def delta_prepare(rows: torch.Tensor, ab: torch.Tensor, taps: torch.Tensor, conv_state: torch.Tensor, step,
@@ -1082,7 +1127,7 @@ def delta_prepare(rows: torch.Tensor, ab: torch.Tensor, taps: torch.Tensor, conv
     _check(library().somi_delta_prepare(
         _ptr(rows), dtype_code(rows.dtype), ctypes.c_int64(rows.stride(0)), _ptr(ab), _ptr(taps), width, _ptr(conv_state),
         _ptr(step.token_entry), _ptr(step.entry_start), _ptr(step.state_slots), _ptr(a_log), _ptr(dt_bias), n, entries,
-        groups, heads, dim, vdim, _ptr(qkv), _ptr(beta), _ptr(decay), _stream()))
+        int(step.max_entry_len), groups, heads, dim, vdim, _ptr(qkv), _ptr(beta), _ptr(decay), _stream()))
     return qkv, beta, decay
 
 
@@ -1137,10 +1182,11 @@ ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, groups: int, keep: int, scores: str = "softmax",
-              normalize: bool = True) -> tuple[torch.Tensor, torch.Tensor]:
+              normalize: bool = True, correction: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """Chosen experts [N, top] int32 and their weights [N, top] float32: float32 scores (``scores``: the softmax over all
     experts, or each expert's own sigmoid), the ``keep`` best of ``groups`` runs of neighbouring experts, the ``top`` best
-    experts of those; weights over their sum (``normalize``) or the scores as they are."""
+    experts of those; weights over their sum (``normalize``) or the scores as they are.  ``correction`` [experts] float32 is
+    added to the scores for the choice, not for the weights."""
     _need(x, "rows")
     n, width = x.shape
     _need(router, "router", torch.float32)
@@ -1148,10 +1194,13 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, groups: int, keep
         raise KernelError(f"moe_route: router {tuple(router.shape)} does not fit rows of {width}")
     if scores not in ROUTER_SCORES:
         raise KernelError(f"moe_route: unknown scores {scores!r}; known: {sorted(ROUTER_SCORES)}")
+    if correction is not None:
+        _need(correction, "choice correction", torch.float32, (router.shape[0],))
     chosen = torch.empty((n, top), dtype=torch.int32, device=x.device)
     weight = torch.empty((n, top), dtype=torch.float32, device=x.device)
     logits = torch.empty((n, router.shape[0]), dtype=torch.float32, device=x.device)     # the router's sums, if it tiles them
-    _check(library().somi_moe_route(_ptr(x), dtype_code(x.dtype), ctypes.c_int64(x.stride(0)), _ptr(router), _ptr(logits), n,
+    _check(library().somi_moe_route(_ptr(x), dtype_code(x.dtype), ctypes.c_int64(x.stride(0)), _ptr(router), _ptr(correction),
+                                    _ptr(logits), n,
                                     width, router.shape[0], int(top), int(groups), int(keep), ROUTER_SCORES[scores],
                                     1 if normalize else 0, _ptr(chosen), _ptr(weight), _stream()))
     return chosen, weight
@@ -1196,6 +1245,36 @@ def moe_gate_up(x: torch.Tensor, gate_up: torch.Tensor, tiles: torch.Tensor, ord
     _check(library().somi_moe_product(_ptr(x), ctypes.c_int64(x.stride(0)), _ptr(gate_up), dtype_code(x.dtype), 1, _ptr(tiles),
                                       tiles.shape[0], _ptr(order), _ptr(input_weight), int(top), two_f // 2, k, ctypes.c_float(limit),
                                       ctypes.c_float(alpha), ctypes.c_float(shift), _ptr(act), _stream()))
+    return act
+
+
+MOE_DOWN, MOE_GATED, MOE_SQUARED_RELU = 0, 1, 2      # what an experts' product does at its end (and whether it gathers rows by token)
+
+
+def moe_up(x: torch.Tensor, up: torch.Tensor, tiles: torch.Tensor, order: torch.Tensor, top: int,
+           tile_rows: int = MOE_TILE_ROWS, mfma: bool = False, input_weight: torch.Tensor | None = None) -> torch.Tensor:
+    """act[p] = relu(W_up[e] x[t])^2 for the sorted pairs p = (t, e), experts without a gate; up: [experts, F, K] ->
+    [pairs, F].  ``input_weight`` as in :func:`moe_gate_up`."""
+    _need(x, "rows")
+    _need(up, "up matrices", x.dtype)
+    experts, f, k = up.shape
+    if x.shape[1] != k:
+        raise KernelError(f"moe_up: matrices {tuple(up.shape)} do not fit rows of {x.shape[1]}")
+    pairs = order.numel()
+    if input_weight is not None:
+        _need(input_weight, "pair weights", torch.float32)
+        if input_weight.numel() != pairs:
+            raise KernelError(f"moe_up: {input_weight.numel()} weights for {pairs} pairs")
+    act = torch.empty((pairs, f), dtype=x.dtype, device=x.device)
+    none = ctypes.c_float(0.0)
+    if mfma:
+        _check(library().somi_moe_product_mfma(_ptr(x), ctypes.c_int64(x.stride(0)), _ptr(up), MOE_SQUARED_RELU, _ptr(tiles),
+                                               tiles.shape[0], int(tile_rows), _ptr(order), _ptr(input_weight), int(top), f, k,
+                                               none, none, none, _ptr(act), _stream()))
+    else:
+        _check(library().somi_moe_product(_ptr(x), ctypes.c_int64(x.stride(0)), _ptr(up), dtype_code(x.dtype), MOE_SQUARED_RELU,
+                                          _ptr(tiles), tiles.shape[0], _ptr(order), _ptr(input_weight), int(top), f, k, none,
+                                          none, none, _ptr(act), _stream()))
     return act
 
 
@@ -1630,7 +1709,131 @@ def mixed_attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.
     return out
 
 
+# ------------------------------------------------------------- heads normed one by one, a gate a head
+def head_norm_store(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tensor | None,
+                    k_weight: torch.Tensor | None, norm_values: bool, eps: float, temperature: tuple[float, int] | None,
+                    heads: int, kv_heads: int, dim: int, vdim: int, k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
+    """From float32 rows [q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim) | ...], possibly columns of wider rows:
+    q and k RMS-normed head by head with weights of a head's size (None: no norm), q times ``1 + coef ln(floor((p + 1) /
+    every) + 1)`` for ``temperature`` (coef, every), v divided by each head's root mean square (``norm_values``); k and v
+    into the tokens' slots of ``k_cache`` [pages, kv_heads, page, padded] and ``v_cache`` [pages, kv_heads, padded, page]
+    -> q [N, heads * padded] in the caches' dtype.  Channels past dim and vdim are zeros."""
+    if not isinstance(rows, torch.Tensor) or not rows.is_cuda or rows.dtype != torch.float32 or rows.dim() != 2 or rows.stride(1) != 1:
+        raise KernelError("head_norm_store: the rows must be a float32 matrix on the GPU with contiguous rows")
+    n = rows.shape[0]
+    if rows.shape[1] < heads * dim + kv_heads * (dim + vdim):
+        raise KernelError(f"head_norm_store: rows of {rows.shape[1]} values do not hold the projections")
+    _need(k_cache, "key pages")
+    if k_cache.dim() != 4 or k_cache.shape[1] != kv_heads:
+        raise KernelError(f"head_norm_store: key pages {tuple(k_cache.shape)} != [pages, {kv_heads}, page, padded]")
+    page, padded = k_cache.shape[2], k_cache.shape[3]
+    _need(v_cache, "value pages", k_cache.dtype, _v_shape(k_cache))
+    _need(positions, "positions", torch.int32, (n,))
+    _need(slots, "slot mapping", torch.int32, (n,))
+    for weight, name in ((q_weight, "q norm weight"), (k_weight, "k norm weight")):
+        if weight is not None:
+            _need(weight, name, torch.float32, (dim,))
+    coef, every = temperature if temperature is not None else (0.0, 1)
+    q = torch.empty((n, heads * padded), dtype=k_cache.dtype, device=rows.device)
+    _check(library().somi_head_norm_store(_ptr(rows), ctypes.c_int64(rows.stride(0)), n, _ptr(positions), _ptr(slots),
+                                          _ptr(q_weight), _ptr(k_weight), 1 if norm_values else 0, ctypes.c_float(eps),
+                                          ctypes.c_float(coef), int(every), int(heads), int(kv_heads), int(dim), int(vdim),
+                                          padded, _ptr(q), _ptr(k_cache), _ptr(v_cache), page, dtype_code(k_cache.dtype),
+                                          _stream()))
+    return q
+
+
+def _rows_out(out: torch.Tensor, n: int, width: int, what: str) -> ctypes.c_int64:
+    """Row stride of a result that may be columns of wider rows."""
+    if not isinstance(out, torch.Tensor) or not out.is_cuda or tuple(out.shape) != (n, width) or out.stride(1) != 1:
+        raise KernelError(f"{what}: the result must be [{n}, {width}] on the GPU with contiguous rows")
+    return ctypes.c_int64(out.stride(0))
+
+
+def head_gate(x: torch.Tensor, gate: torch.Tensor | None, heads: int, vdim: int, scale: float, out: torch.Tensor) -> None:
+    """out[t, h, :] = scale * x[t, h, :vdim] * sigmoid(gate[t, h]) for x [N, heads * padded]; gate: float32 [N, heads],
+    possibly columns of wider rows (None: no gate); out: [N, heads * vdim], likewise."""
+    _need(x, "gated rows")
+    n = x.shape[0]
+    if x.shape[1] % heads or x.shape[1] // heads < vdim or out.dtype != x.dtype:
+        raise KernelError(f"head_gate: rows of {x.shape[1]} {x.dtype} do not hold {heads} heads of {vdim} for a result in {out.dtype}")
+    stride = 0
+    if gate is not None:
+        if not gate.is_cuda or gate.dtype != torch.float32 or tuple(gate.shape) != (n, heads) or gate.stride(1) != 1:
+            raise KernelError(f"head_gate: the gate is float32 rows of {heads} values on the GPU")
+        stride = gate.stride(0)
+    _check(library().somi_head_gate(_ptr(x), dtype_code(x.dtype), _ptr(gate), ctypes.c_int64(stride), ctypes.c_float(scale), n,
+                                    int(heads), x.shape[1] // heads, int(vdim), _ptr(out),
+                                    _rows_out(out, n, heads * vdim, "head_gate"), _stream()))
+
+
+# ------------------------------------------------------------------------------------------ state-space duality, minGRU
+def _float_rows(t: torch.Tensor, n: int, width: int, name: str) -> ctypes.c_int64:
+    if not isinstance(t, torch.Tensor) or not t.is_cuda or t.dtype != torch.float32 or tuple(t.shape) != (n, width) or t.stride(1) != 1:
+        raise KernelError(f"{name}: must be float32 [{n}, {width}] on the GPU with contiguous rows")
+    return ctypes.c_int64(t.stride(0))
+
+
+def ssd_scan(xbc: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor,
+             entry_start: torch.Tensor, state_slots: torch.Tensor, state: torch.Tensor, groups: int) -> torch.Tensor:
+    """S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + D x per head with dt = softplus(raw + dt_bias) -> y [N, heads * P]
+    float32.  xbc: [N, heads * P + 2 groups * N_state] float32, x then B then C; raw_dt: [N, heads] float32, possibly
+    columns of wider rows; state: [slots, heads, P, N_state] float32, read and written in place."""
+    _need(state, "recurrent state", torch.float32)
+    _, heads, p, n_state = state.shape
+    n = xbc.shape[0]
+    _need(xbc, "x, B and C", torch.float32, (n, heads * p + 2 * groups * n_state))
+    stride = _float_rows(raw_dt, n, heads, "dt rows")
+    for t, name in ((dt_bias, "dt bias"), (a_log, "decay rates"), (skip, "skip weights")):
+        _need(t, name, torch.float32, (heads,))
+    entries = state_slots.numel()
+    _need(entry_start, "entry offsets", torch.int32, (entries + 1,))
+    _need(state_slots, "state slots", torch.int32, (entries,))
+    y = torch.empty((n, heads * p), dtype=torch.float32, device=xbc.device)
+    _check(library().somi_ssd_scan(_ptr(xbc), _ptr(raw_dt), stride, _ptr(dt_bias), _ptr(a_log), _ptr(skip), _ptr(entry_start),
+                                   _ptr(state_slots), _ptr(state), entries, heads, int(groups), p, n_state, _ptr(y), _stream()))
+    return y
+
+
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, scale: float,
+                     out: torch.Tensor) -> None:
+    """out = scale * weight * (y silu(z)), each of ``groups`` equal parts of a row divided by its own root mean square.  y:
+    [N, width] float32; z: float32, possibly columns of wider rows; out: [N, width], likewise."""
+    _need(y, "rows", torch.float32)
+    n, width = y.shape
+    _need(weight, "norm weight", torch.float32, (width,))
+    _check(library().somi_gated_group_norm(_ptr(y), _ptr(z), _float_rows(z, n, width, "gate rows"), _ptr(weight), int(groups),
+                                           ctypes.c_float(eps), ctypes.c_float(scale), n, width, _ptr(out),
+                                           _rows_out(out, n, width, "gated_group_norm"), dtype_code(out.dtype), _stream()))
+
+
+def min_gru(rows: torch.Tensor, z_bias: torch.Tensor, x_bias: torch.Tensor, step, state: torch.Tensor, scale: float,
+            out: torch.Tensor) -> None:
+    """S <- (1 - z) S + z c element by element with z = sigmoid(rz + z_bias), u = rx + x_bias, c = u + 1/2 (u >= 0) or
+    sigmoid(u); out = scale * S * silu(rg).  rows: [N, rz | rx | rg] float32, possibly columns of wider rows; state:
+    [slots, width] float32, read and written in place; out: [N, width], likewise columns."""
+    _need(state, "recurrent state", torch.float32)
+    width = state.shape[1]
+    n = rows.shape[0]
+    stride = _float_rows(rows, n, 3 * width, "minGRU rows")
+    _need(z_bias, "gate bias", torch.float32, (width,))
+    _need(x_bias, "candidate bias", torch.float32, (width,))
+    entries = step.state_slots.numel()
+    _need(step.entry_start, "entry offsets", torch.int32, (entries + 1,))
+    _check(library().somi_min_gru(_ptr(rows), stride, _ptr(z_bias), _ptr(x_bias), _ptr(step.entry_start), _ptr(step.state_slots),
+                                  _ptr(state), entries, int(step.max_entry_len), width, ctypes.c_float(scale), _ptr(out),
+                                  _rows_out(out, n, width, "min_gru"), dtype_code(out.dtype), _stream()))
+
+
 # ------------------------------------------------------------------------------------------ activations and gates
+def squared_relu(z: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """relu(z)^2 of float32 values, in ``out_dtype``."""
+    _need(z, "rows", torch.float32)
+    out = torch.empty(z.shape, dtype=out_dtype, device=z.device)
+    _check(library().somi_squared_relu(_ptr(z), _ptr(out), dtype_code(out_dtype), ctypes.c_int64(z.numel()), _stream()))
+    return out
+
+
 def xielu(z: torch.Tensor, pq: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
     """softplus(p) z^2 + z / 2 for z > 0 and (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 otherwise; z: float32; pq: the
     two stored numbers, float32 on the device."""

@@ -8,6 +8,8 @@ from .kamedra import kamedra_plan
 from .metitar import metitar_plan
 from .qwen2 import qwen2_plan
 from .rusolorn import rusolorn_plan
+from .tomopel import tomopel_plan
 
 __all__ = ["DecoderModel", "LayerSpec", "ModelPlan", "collect_weight_specs", "load_model",
-           "gizilorn_plan", "kamedra_plan", "make_runner", "metitar_plan", "make_runtime", "qwen2_plan", "random_model", "rusolorn_plan"]
+           "gizilorn_plan", "kamedra_plan", "make_runner", "metitar_plan", "make_runtime", "qwen2_plan", "random_model", "rusolorn_plan",
+           "tomopel_plan"]

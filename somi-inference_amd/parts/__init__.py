@@ -3,6 +3,7 @@
 from .attention import GroupedQueryAttention
 from .base import (PAGE, Block, BorrowedCache, CompositeSpec, FeedForward, FixedStateSpec, LayerCache, Mixer, Norm, PagedKVSpec, PagedSpec,
                    PageTensor, Part, PartSpec, PositionEncoding, Runtime)
+from .biased_attention import BiasedAttention
 from .block import HyperConnectionBlock, OutputNormBlock, ParallelBlock, PreNormBlock
 from .delta_rule import GatedDeltaRule
 from .diff_attention import DifferentialAttention
@@ -12,6 +13,8 @@ from .gla import GatedLinearAttention
 from .hgrn2 import HGRN2
 from .input_conv import ShortConvInput
 from .latent_attention import LatentAttention
+from .mamba2 import Mamba2
+from .min_gru import MinGRU
 from .mixed_attention import MixedHeadsAttention
 from .moe import RoutedExperts
 from .norm import DynamicTanh, LayerNorm, RMSNorm
@@ -19,6 +22,7 @@ from .parallel_mixer import ParallelMixers
 from .position import NoPosition, RotaryPosition
 from .registry import build_part, part_kinds, register_part, unregister_part
 from .residual import ResidualStream
+from .rows_mixer import RowsMixer
 from .token_input import GatedTokenInput
 
 register_part("norm", "rmsnorm", RMSNorm)
@@ -34,6 +38,9 @@ register_part("mixer", "parallel", ParallelMixers)
 register_part("mixer", "latent_attention", LatentAttention)
 register_part("mixer", "hgrn2", HGRN2)
 register_part("mixer", "mixed_heads_attention", MixedHeadsAttention)
+register_part("mixer", "biased_attention", BiasedAttention)
+register_part("mixer", "mamba2", Mamba2)
+register_part("mixer", "min_gru", MinGRU)
 register_part("feed_forward", "swiglu", SwiGLU)
 register_part("feed_forward", "routed_experts", RoutedExperts)
 register_part("feed_forward", "poly_norm", PolyNormFF)
@@ -48,7 +55,7 @@ register_part("embedding", "token_embedding", TokenEmbedding)
 register_part("head", "lm_head", LMHead)
 
 __all__ = [
-    "ActivatedFF", "Block", "BorrowedCache", "HyperConnectionBlock", "MixedHeadsAttention", "CompositeSpec", "HGRN2", "LatentAttention", "LayerNorm", "OutputNormBlock", "PolyNormFF", "ShortConvInput", "DifferentialAttention", "DynamicTanh", "GatedDeltaRule", "GatedTokenInput", "ParallelBlock", "ParallelMixers", "RoutedExperts", "FeedForward", "FixedStateSpec", "GatedLinearAttention", "GroupedQueryAttention", "LMHead", "LayerCache", "Mixer",
+    "ActivatedFF", "BiasedAttention", "Mamba2", "MinGRU", "RowsMixer", "Block", "BorrowedCache", "HyperConnectionBlock", "MixedHeadsAttention", "CompositeSpec", "HGRN2", "LatentAttention", "LayerNorm", "OutputNormBlock", "PolyNormFF", "ShortConvInput", "DifferentialAttention", "DynamicTanh", "GatedDeltaRule", "GatedTokenInput", "ParallelBlock", "ParallelMixers", "RoutedExperts", "FeedForward", "FixedStateSpec", "GatedLinearAttention", "GroupedQueryAttention", "LMHead", "LayerCache", "Mixer",
     "NoPosition", "Norm", "PAGE", "PageTensor", "PagedKVSpec", "PagedSpec", "Part", "PartSpec", "PositionEncoding", "PreNormBlock", "RMSNorm",
     "ResidualStream", "RotaryPosition", "Runtime", "SwiGLU", "TokenEmbedding", "build_part", "part_kinds",
     "register_part", "unregister_part",

@@ -166,11 +166,11 @@ class HyperConnectionBlock(Block):
     """A pre-norm layer around ``streams`` residual streams instead of one.  For sublayer q (the mixer, then the
     feed-forward) with its three tensors ``in`` [S], ``mix`` [S, S] (from, to) and ``out`` [S]:
 
-        u = sum_s in[s] x_s;     y = sublayer(norm_q(u));     x_t <- sum_s mix[s, t] x_s + out[t] y    (all t at once).
+        u = sum_s in[s] x_s;     y = sublayer(norm_q(u));     x_t <- sum_s mix[s, t] x_s + m out[t] y    (all t at once)
 
-    The streams are all equal to the embedded rows when the first such layer meets them, and what the model's final
+    with m = ``residual_mult``.  The streams are all equal to the embedded rows when the first such layer meets them, and what the model's final
     norm reads is their sum.  ``connections`` False: no such tensors; one stream with in = mix = out = 1, the plain
-    residual sum.  Streams, their sums and the norms are float32; a sublayer's last product is computed into float32
+    residual sum (of m times the sublayers' outputs).  Streams, their sums and the norms are float32; a sublayer's last product is computed into float32
     rows, and one kernel does a sublayer's write and the next sublayer's read and norm.  A layer without a feed-forward
     has the first sublayer only.  ``names``: the sub-prefixes of the two norms, the mixer, the feed-forward and the two
     sets of connection tensors."""
@@ -179,13 +179,13 @@ class HyperConnectionBlock(Block):
                      "mixer_streams": "hc1", "ffn_streams": "hc2"}
 
     def __init__(self, prefix: str, mixer: PartSpec, feed_forward: PartSpec | None, mixer_norm: PartSpec,
-                 ffn_norm: PartSpec | None = None, streams: int = 1, connections: bool = True,
+                 ffn_norm: PartSpec | None = None, streams: int = 1, connections: bool = True, residual_mult: float = 1.0,
                  names: dict[str, str] | None = None) -> None:
         super().__init__(prefix)
         sub = dict(self.DEFAULT_NAMES)
         sub.update(names or {})
         self.sub = sub
-        self.streams, self.connections = int(streams), bool(connections)
+        self.streams, self.connections, self.residual_mult = int(streams), bool(connections), float(residual_mult)
         if not 1 <= self.streams <= ops.HC_MAX_STREAMS or (not self.connections and self.streams != 1):
             raise ValueError(f"{prefix}: 1 to {ops.HC_MAX_STREAMS} streams (one without connection tensors), got {streams}")
         self.mixer_norm = build_part("norm", mixer_norm, prefix=self.name(sub["mixer_norm"]))
@@ -221,10 +221,10 @@ class HyperConnectionBlock(Block):
         super().load(fetch, runtime)
         self.links = []
         for base in self._connection_names():
-            self.links.append((fetch(f"{base}.in"), fetch(f"{base}.mix").contiguous(), fetch(f"{base}.out")))
+            self.links.append((fetch(f"{base}.in"), fetch(f"{base}.mix").contiguous(), fetch(f"{base}.out") * self.residual_mult))
         if not self.connections:
             one = torch.ones((1,), dtype=torch.float32, device=runtime.device)
-            self.links = [(one, one.view(1, 1), one)] * 2
+            self.links = [(one, one.view(1, 1), one * self.residual_mult)] * 2
 
     def forward(self, stream: ResidualStream, step, cache: LayerCache | None) -> None:
         lanes = stream.fan_out(self.streams)

@@ -1,13 +1,15 @@
-"""Mixture of experts: a router picks a few small gated feed-forwards per token; a shared one may run for all.
+"""Mixture of experts: a router picks a few small feed-forwards per token; a shared one may run for all.
 
 Router: ``z = W_r x`` in float32 and scores ``s = softmax(z)`` over all experts, or ``s = sigmoid(z)`` expert by expert
 (``scores``).  The experts come in ``groups`` equal runs of neighbours; a run scores as its best expert, and only
 experts of the ``keep`` best runs can be chosen.  Of those the ``top`` with the largest s are taken, weighted by s over
-the sum of the chosen scores (+ 1e-20) or by s as it is (``normalize``).  An expert is
+the sum of the chosen scores (+ 1e-20) or by s as it is (``normalize``).  With a ``correction`` tensor, one number an
+expert, the choice looks at s + correction and the weights at s alone.  A gated expert is
 
     g = min(W_gate x, limit);  u = clamp(W_up x, -limit, limit);  y = W_down (g sigmoid(alpha g) (u + shift))
 
-without biases (no ``limit``, alpha 1 and shift 0: the plain ``silu(W_gate x) * (W_up x)``); the output is the weighted
+without biases (no ``limit``, alpha 1 and shift 0: the plain ``silu(W_gate x) * (W_up x)``); one without a gate (``unit``
+"squared_relu") is ``y = W_down relu(W_up x)^2``.  The output is the weighted
 sum of the chosen experts' outputs or, with ``weight_on="input"``, the sum of the experts applied to ``w x`` (the
 weight then scales the float32 sums of gate and up before the unit, which is not the same thing since the unit is not
 linear); plus the shared expert's (the same form with sizes and a limit of its own).  The (token, expert) pairs are sorted by expert on the device, so that an
@@ -20,7 +22,7 @@ import torch
 
 from ..kernels import ops
 from ..kernels.stages import stage
-from ..weights.spec import MATRIX, VECTOR, WeightSpec
+from ..weights.spec import MATRIX, VECTOR, Init, WeightSpec
 from .base import FeedForward, Fetch, Runtime
 from .linear import Projection
 
@@ -38,17 +40,20 @@ class ClampedGLU:
 class RoutedExperts(FeedForward):
     graph_safe = True
 
-    ROLES = {"router": "router", "expert": "e", "shared": "shared", "gate": "gate", "up": "up", "down": "down"}
+    ROLES = {"router": "router", "expert": "e", "shared": "shared", "gate": "gate", "up": "up", "down": "down",
+             "correction": "correction"}
 
+    UNITS = ("clamped_glu", "squared_relu")
     SCORES = ("softmax", "sigmoid")
     WEIGHT_ON = ("output", "input")
 
-    def __init__(self, prefix: str, hidden_size: int, num_experts: int, top: int, expert_size: int, limit: float | None,
+    def __init__(self, prefix: str, hidden_size: int, num_experts: int, top: int, expert_size: int, limit: float | None = None,
                  groups: int = 1, keep_groups: int = 1, shared_size: int | None = None, shared_limit: float | None = None,
                  alpha: float = 1.702, shift: float = 1.0, names: dict[str, str] | None = None, suffix: str = "weight",
-                 scores: str = "softmax", normalize: bool = True, weight_on: str = "output") -> None:
-        """``names``: ``router``, the experts' stem (``e`` gives ``e0``, ``e1``, ...), ``shared``, and the three matrices
-        of an expert; ``suffix`` follows a matrix's name (empty: nothing)."""
+                 scores: str = "softmax", normalize: bool = True, weight_on: str = "output", unit: str = "clamped_glu",
+                 correction: bool = False) -> None:
+        """``names``: ``router``, the experts' stem (``e`` gives ``e0``, ``e1``, ...), ``shared``, the three matrices
+        of an expert (two without a gate) and ``correction``; ``suffix`` follows a matrix's name (empty: nothing)."""
         super().__init__(prefix)
         unknown = set(names or {}) - set(self.ROLES)
         if unknown:
@@ -65,6 +70,9 @@ class RoutedExperts(FeedForward):
         if scores not in self.SCORES or weight_on not in self.WEIGHT_ON:
             raise ValueError(f"{prefix}: scores {scores!r} (one of {self.SCORES}), weight_on {weight_on!r} (one of {self.WEIGHT_ON})")
         self.scores, self.normalize, self.weight_on = scores, bool(normalize), weight_on
+        if unit not in self.UNITS:
+            raise ValueError(f"{prefix}: an expert's unit is one of {self.UNITS}, got {unit!r}")
+        self.gated, self.has_correction = unit == "clamped_glu", bool(correction)
         self.unit = ClampedGLU(limit, alpha, shift)
         self.shared_size = int(shared_size) if shared_size else None
         self.shared_unit = ClampedGLU(shared_limit if shared_limit is not None else limit, alpha, shift) if self.shared_size else None
@@ -76,39 +84,44 @@ class RoutedExperts(FeedForward):
     def _expert(self, index: int) -> str:
         return f"{self.names['expert']}{index}"
 
+    def _ups(self) -> tuple[str, ...]:
+        """The matrices in front of an expert's unit."""
+        return ("gate", "up") if self.gated else ("up",)
+
     def weight_specs(self) -> list[WeightSpec]:
-        h, f = self.hidden_size, self.expert_size
+        h = self.hidden_size
         specs = [WeightSpec(self._matrix(self.names["router"]), (self.num_experts, h), VECTOR)]
-        for e in range(self.num_experts):
-            specs += [WeightSpec(self._matrix(self._expert(e), self.names["gate"]), (f, h), MATRIX),
-                      WeightSpec(self._matrix(self._expert(e), self.names["up"]), (f, h), MATRIX),
-                      WeightSpec(self._matrix(self._expert(e), self.names["down"]), (h, f), MATRIX)]
+        if self.has_correction:
+            specs.append(WeightSpec(self.name(self.names["correction"]), (self.num_experts,), VECTOR, Init(0.0, 0.02)))
+        feeds = [(self._expert(e), self.expert_size) for e in range(self.num_experts)]
         if self.shared_size:
-            s = self.names["shared"]
-            specs += [WeightSpec(self._matrix(s, self.names["gate"]), (self.shared_size, h), MATRIX),
-                      WeightSpec(self._matrix(s, self.names["up"]), (self.shared_size, h), MATRIX),
-                      WeightSpec(self._matrix(s, self.names["down"]), (h, self.shared_size), MATRIX)]
+            feeds.append((self.names["shared"], self.shared_size))
+        for feed, size in feeds:
+            specs += [WeightSpec(self._matrix(feed, self.names[role]), (size, h), MATRIX) for role in self._ups()]
+            specs.append(WeightSpec(self._matrix(feed, self.names["down"]), (h, size), MATRIX))
         return specs
 
     def load(self, fetch: Fetch, runtime: Runtime) -> None:
         super().load(fetch, runtime)
         self.router = fetch(self._matrix(self.names["router"]))            # float32: the router is computed in 32-bit
-        gate_up, down = [], []
+        self.correction = fetch(self.name(self.names["correction"])) if self.has_correction else None
+        up, down = [], []
         for e in range(self.num_experts):
-            gate_up.append(torch.cat([fetch(self._matrix(self._expert(e), self.names[role])) for role in ("gate", "up")], dim=0))
+            up.append(torch.cat([fetch(self._matrix(self._expert(e), self.names[role])) for role in self._ups()], dim=0))
             down.append(fetch(self._matrix(self._expert(e), self.names["down"])))
-        self.gate_up = torch.stack(gate_up).contiguous()                  # [experts, 2 F, H], gate rows first
+        self.up = torch.stack(up).contiguous()                            # [experts, (2) F, H], gate rows first
         self.down = torch.stack(down).contiguous()                        # [experts, H, F]
-        self.shared_gate_up = self.shared_down = None
+        self.shared_up = self.shared_down = None
         if self.shared_size:
             s = self.names["shared"]
-            self.shared_gate_up = Projection.stacked([fetch(self._matrix(s, self.names[role])) for role in ("gate", "up")],
-                                                     label="shared gate_up")
+            self.shared_up = Projection.stacked([fetch(self._matrix(s, self.names[role])) for role in self._ups()],
+                                                label="shared gate_up" if self.gated else "shared up")
             self.shared_down = Projection(fetch(self._matrix(s, self.names["down"])), label="shared down")
 
     def flops(self, tokens: int, attended: int) -> float:
-        routed = 6.0 * tokens * self.top * self.expert_size * self.hidden_size
-        shared = 6.0 * tokens * (self.shared_size or 0) * self.hidden_size
+        matrices = len(self._ups()) + 1
+        routed = 2.0 * matrices * tokens * self.top * self.expert_size * self.hidden_size
+        shared = 2.0 * matrices * tokens * (self.shared_size or 0) * self.hidden_size
         return routed + shared + 2.0 * tokens * self.num_experts * self.hidden_size
 
     def forward(self, x, step=None) -> torch.Tensor:
@@ -116,23 +129,32 @@ class RoutedExperts(FeedForward):
             x = x.materialize()
         with stage("router"):
             chosen, weight = ops.moe_route(x, self.router, self.top, self.groups, self.keep_groups, self.scores,
-                                           self.normalize)
+                                           self.normalize, self.correction)
             # bfloat16: the products run on the matrix cores, in tiles sized by the rows an expert gets in this step
-            mfma = ops.moe_mfma_supported(x, self.gate_up, self.down)
+            mfma = ops.moe_mfma_supported(x, self.up, self.down)
             rows = ops.moe_tile_rows(chosen.numel(), self.num_experts, mfma)
             order, _, tiles = ops.moe_align(chosen, self.num_experts, rows)
-        with stage("experts gate_up"):
-            act = ops.moe_gate_up(x, self.gate_up, tiles, order, self.top, self.unit.limit, self.unit.alpha, self.unit.shift,
-                                  tile_rows=rows, mfma=mfma, input_weight=weight if self.weight_on == "input" else None)
+        input_weight = weight if self.weight_on == "input" else None
+        with stage("experts gate_up" if self.gated else "experts up"):
+            if self.gated:
+                act = ops.moe_gate_up(x, self.up, tiles, order, self.top, self.unit.limit, self.unit.alpha, self.unit.shift,
+                                      tile_rows=rows, mfma=mfma, input_weight=input_weight)
+            else:
+                act = ops.moe_up(x, self.up, tiles, order, self.top, tile_rows=rows, mfma=mfma, input_weight=input_weight)
         with stage("experts down"):
             pairs = ops.moe_down(act, self.down, tiles, order, weight if self.weight_on == "output" else None, self.top,
                                  tile_rows=rows, mfma=mfma)
-        shared = None
-        if self.shared_size:
-            unit = self.shared_unit
-            gate_up = self.shared_gate_up(x)
-            with stage("activation"):
-                gated = ops.clamped_glu(gate_up, unit.limit, unit.alpha, unit.shift)
-            shared = self.shared_down(gated)
+        shared = self._shared(x) if self.shared_size else None
         with stage("experts' sum"):
             return ops.moe_combine(pairs, self.top, shared)
+
+    def _shared(self, x: torch.Tensor) -> torch.Tensor:
+        if not self.gated:
+            up = self.shared_up(x, torch.float32)
+            with stage("activation"):
+                act = ops.squared_relu(up, self.runtime.dtype)
+            return self.shared_down(act, torch.float32)
+        gate_up = self.shared_up(x)
+        with stage("activation"):
+            gated = ops.clamped_glu(gate_up, self.shared_unit.limit, self.shared_unit.alpha, self.shared_unit.shift)
+        return self.shared_down(gated)

@@ -16,13 +16,15 @@ class RMSNorm(Norm):
     fusable = True        # weight * (h / sqrt(mean(h^2) + eps)): what a projection can apply while it loads h
 
     def __init__(self, prefix: str, hidden_size: int, eps: float,
-                 init: tuple[float, float] = (1.0, 0.1), tensor: str = "weight") -> None:
-        """``tensor``: what the checkpoint calls the scale under the part's prefix."""
+                 init: tuple[float, float] = (1.0, 0.1), tensor: str = "weight", around_one: bool = False) -> None:
+        """``tensor``: what the checkpoint calls the scale under the part's prefix.  ``around_one``: what is stored is
+        what the scale adds to one (the sum is made once, in float32)."""
         super().__init__(prefix)
         self.tensor = str(tensor)
         self.hidden_size = int(hidden_size)
         self.eps = float(eps)
-        self._init = Init(*init)
+        self.around_one = bool(around_one)
+        self._init = Init(init[0] - 1.0, init[1]) if self.around_one else Init(*init)
         self.weight: torch.Tensor | None = None
 
     def weight_specs(self) -> list[WeightSpec]:
@@ -31,6 +33,8 @@ class RMSNorm(Norm):
     def load(self, fetch: Fetch, runtime: Runtime) -> None:
         super().load(fetch, runtime)
         self.weight = fetch(self.name(self.tensor))
+        if self.around_one:
+            self.weight = (self.weight + 1.0).contiguous()
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         return ops.rmsnorm(h, self.weight, self.eps, self.runtime.dtype)
