@@ -118,6 +118,7 @@ class PartEngine:
         from somi_inference_amd.cache import CacheManager
         self.mixers, self.dtype, self.device = list(mixers), dtype, device
         needs = [(borrow or {}).get(i, m.cache_spec()) for i, m in enumerate(self.mixers)]
+        self.splits = tuple(sorted({m.entry_split for m in self.mixers if m.entry_split is not None}))
         self.cache = CacheManager(needs, block_size=block_size, num_blocks=num_blocks, max_requests=max_requests,
                                   dtype=dtype, device=device)
 
@@ -130,7 +131,7 @@ class PartEngine:
                 self.cache.register(rid)
             self.cache.reserve(rid, x.shape[0])
             entries.append(StepEntry(rid, [0] * x.shape[0], []))
-        step = build_step(entries, self.cache, self.device, ())
+        step = build_step(entries, self.cache, self.device, self.splits)
         rows = torch.cat([x for _, x in portions]).to(self.dtype).to(self.device).contiguous()
         outs = []
         for index, mixer in enumerate(self.mixers):
