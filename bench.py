@@ -228,6 +228,63 @@ def gizilorn_closest_attention_config_dict(sizes: str) -> dict:
             "use_sliding_window": True, "sliding_window": window, "max_window_layers": 0}
 
 
+# layer sizes of Tomopel models that resemble real ones: (width, residual streams, attention heads, key/value heads, head
+# size, recurrent heads, their value size, their state, groups of B and C, taps, minGRU width, experts, experts a token, an
+# expert's size, the shared expert's size, the dense feed-forward's size, vocabulary).  Six layers: attention beside
+# Mamba-2 in all but the fourth, which is a minGRU; a dense feed-forward in the first, routed experts in the others.
+TOMOPEL_SIZES = {
+    "1b": (2048, 2, 16, 4, 128, 32, 64, 128, 1, 4, 2048, 32, 4, 512, 1024, 4096, 32000),
+    "7b": (4096, 2, 32, 8, 128, 64, 64, 128, 1, 4, 4096, 64, 6, 1024, 2048, 8192, 32000),
+}
+TOMOPEL_LAYERS, TOMOPEL_PARALLEL = 6, 5
+
+
+def tomopel_config_dict(sizes: str) -> dict:
+    (width, streams, heads, kv_heads, dim, r_heads, r_vdim, state, groups, taps, gru, experts, top, ff, shared, dense_ff,
+     vocab) = TOMOPEL_SIZES[sizes]
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}, "shared": {"ff": shared}}
+
+    def parallel(mlp):
+        return {"type": "parallel", "mlp": mlp, "mixer": {
+            "left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "bias_max": 128,
+                     "buckets": 32, "q_temp": {"coef": 0.1, "every": 8192}},
+            "right": {"heads": r_heads, "vdim": r_vdim, "state": state, "groups": groups, "conv": taps, "norm_groups": 1},
+            "left_scale": 0.5, "right_scale": 0.5}}
+    return {"architecture": "Tomopel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "residual_mult": 0.5, "streams": streams,
+            "layers": [parallel({"kind": "dense", "ff": dense_ff}), parallel(moe), parallel(moe),
+                       {"type": "mingru", "mixer": {"width": gru}, "mlp": moe}, parallel(moe), parallel(moe)]}
+
+
+def tomopel_closest_config_dict(sizes: str) -> dict:
+    """The closest model the engine had before: a Rusolorn model of the same width, attention heads (its window holds every
+    context measured here), recurrent state (as many elements a token and layer, in 128 x 128 heads), experts and layers;
+    no token input."""
+    (width, streams, heads, kv_heads, dim, r_heads, r_vdim, state, groups, taps, gru, experts, top, ff, shared, dense_ff,
+     vocab) = TOMOPEL_SIZES[sizes]
+    delta_heads = r_heads * r_vdim * state // (128 * 128)
+    layer = {"type": "parallel",
+             "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                                "mask": {"size": 65536}},
+                       "right": {"heads": delta_heads, "kv_heads": delta_heads // 2, "dim": 128, "vdim": 128, "conv": taps}},
+             "mlp": {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff, "limit": 7.0},
+                     "shared": {"ff": shared, "limit": 7.0}}}
+    return {"architecture": "Rusolorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "residual_mult": 0.5, "layers": [layer] * TOMOPEL_LAYERS}
+
+
+def tomopel_closest_streams_config_dict(sizes: str) -> dict:
+    """The closest model for what stands between the sublayers and for the dense feed-forward: a Gizilorn model of the
+    same width and number of streams, with attention with mixed heads and dense feed-forwards of the same size."""
+    (width, streams, heads, kv_heads, dim, r_heads, r_vdim, state, groups, taps, gru, experts, top, ff, shared, dense_ff,
+     vocab) = TOMOPEL_SIZES[sizes]
+    layer = {"type": "attention", "mlp": {"kind": "dense", "ff": dense_ff},
+             "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                       "mask": {"size": 512}, "rot": {"base": 10000.0, "dims": dim}}}
+    return {"architecture": "Gizilorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "streams": streams,
+            "layers": [layer] * TOMOPEL_LAYERS}
+
+
 # keys of a config.json that name sizes, in the order they are reported under "config" (flat, at most 20 keys)
 SIZE_KEYS = ("hidden_size", "intermediate_size", "num_attention_heads", "num_key_value_heads", "head_dim",
              "vocab_size", "tie_word_embeddings")
@@ -277,6 +334,11 @@ def parse_args() -> argparse.Namespace:
                         "streams, attention with mixed heads, windowed attention over a shared latent) at these layer "
                         "sizes, beside a Metitar model of equal width, latent and feed-forwards and a Qwen2.5-style model "
                         "of equal width, heads and window, each with its stage times")
+    p.add_argument("--tomopel", default=None, choices=sorted(TOMOPEL_SIZES), metavar="SIZES",
+                   help="instead of the default workload: prefill and decode of a Tomopel model (attention with a distance "
+                        "bias beside Mamba-2, minGRU, ungated experts, several residual streams) at these layer sizes, "
+                        "beside a Rusolorn model of equal width, heads, state, experts and layers and a Gizilorn model of "
+                        "equal width, streams and dense feed-forward, each with its stage times")
     p.add_argument("--serving", type=int, default=0, metavar="REQUESTS",
                    help="also run this many requests (prompts of 128 to 2,048 tokens, 256 new tokens each) through "
                         "the scheduler with portions of 512, and report it under 'serving'")
@@ -918,6 +980,89 @@ def run_gizilorn(args) -> dict:
     return out
 
 
+def run_tomopel(args) -> dict:
+    """Prefill and decode of a Tomopel model beside the closest models the engine had, with the stage times of all three
+    and what the attention, recurrence, expert and stream kernels reach of the machine."""
+    (width, streams, heads, kv_heads, dim, r_heads, r_vdim, state, groups, taps, gru, experts, top, ff, shared, dense_ff,
+     vocab) = TOMOPEL_SIZES[args.tomopel]
+    batches, context, tokens = (8, 64), args.context, args.prefill_tokens
+    out: dict = {}
+    for label, config_dict in (("tomopel", tomopel_config_dict(args.tomopel)), ("closest", tomopel_closest_config_dict(args.tomopel)),
+                               ("closest_streams", tomopel_closest_streams_config_dict(args.tomopel))):
+        bench = Workbench(config_dict, dtype=args.dtype, seed=args.seed, block_size=args.block_size,
+                          pool_tokens=Workbench.pool_tokens(batches, context, tokens), max_requests=max(batches))
+        block: dict = {"prefill": {str(n): bench.prefill_run(n) for n in sorted({512, tokens})}}
+        for batch in batches:
+            run = bench.decode_run(batch, max(POINT_MIN_STEPS, args.steps // 2), max(2, args.warmup // 2), context)
+            block[f"decode_b{batch}"] = {"tok_s": round(run["tok_s"], 1), "ms": round(run["ms"], 4),
+                                        "mean_ctx": round(run["mean_ctx"], 1)}
+        block["stages"] = bench.stage_run(tokens, batches[0], context)
+        print_stage_tables(block["stages"])
+        out[label] = block
+        bench.close()
+    bf16_peak = PEAK_FLOPS["bfloat16"]
+    pairs = tokens * (tokens + 1) // 2
+    layers, mixed, routed = TOMOPEL_LAYERS, TOMOPEL_PARALLEL, TOMOPEL_LAYERS - 1
+
+    def stage_ms(block, run, *names):
+        return sum(block["stages"][run].get(name, {}).get("ms", 0.0) for name in names)
+
+    def rate(flops, ms):
+        return {"ms": round(ms, 4), "tflops": round(flops / 1e9 / max(ms, 1e-9), 2),
+                "frac_of_peak": round(flops / 1e3 / max(ms, 1e-9) / bf16_peak * 1e6, 5)}
+
+    def stream(bytes_, ms):
+        return {"ms": round(ms, 4), "gbs": round(bytes_ / 1e6 / max(ms, 1e-9), 1)}
+    run = f"prefill_{tokens}"
+    inner = r_heads * r_vdim
+    channels = inner + 2 * groups * state
+    delta_heads = inner * state // (128 * 128)
+    out["prefill_kernels"] = {
+        "tokens": tokens,
+        "tomopel_attention": rate(mixed * 4.0 * heads * dim * pairs, stage_ms(out["tomopel"], run, "attention")),
+        "closest_attention": rate(layers * 4.0 * heads * dim * pairs, stage_ms(out["closest"], run, "attention")),
+        # per token and element of the state: its update and its product with C here (two passes), three in the closest model
+        "tomopel_recurrence": rate(mixed * 4.0 * inner * state * tokens, stage_ms(out["tomopel"], run, "recurrence")),
+        "closest_recurrence": rate(layers * 6.0 * delta_heads * 128 * 128 * tokens, stage_ms(out["closest"], run, "recurrence")),
+        # three float32 rows read, one row written in the compute dtype
+        "tomopel_gated_recurrence": stream(tokens * gru * (12.0 + 2), stage_ms(out["tomopel"], run, "gated recurrence")),
+        # x, B and C read and written in float32 (the closest model's stage reads bfloat16 rows and norms q and k as well)
+        "tomopel_convolution": stream(mixed * tokens * channels * 8.0, stage_ms(out["tomopel"], run, "convolution")),
+        "closest_convolution": stream(layers * tokens * 2 * delta_heads * 128 * 6.0, stage_ms(out["closest"], run, "convolution, unit norms")),
+        # y and z read in float32, the normed rows written
+        "tomopel_gate_norm": stream(mixed * tokens * inner * 10.0, stage_ms(out["tomopel"], run, "gate, norm")),
+        "closest_gate_norm": stream(layers * tokens * delta_heads * 128 * 8.0, stage_ms(out["closest"], run, "norm, gate")),
+        # the q/k/v sums read, q, k and v written (the closest model's rows are bfloat16)
+        "tomopel_head_norms": stream(mixed * tokens * (heads + 2 * kv_heads) * dim * 6.0, stage_ms(out["tomopel"], run, "head norms, k/v into pages")),
+        "closest_qk_norm": stream(layers * tokens * ((heads + kv_heads) * dim * 4.0 + kv_heads * dim * 2.0), stage_ms(out["closest"], run, "q/k norm, k/v into pages")),
+        "tomopel_experts": rate(routed * 4.0 * tokens * top * ff * width, stage_ms(out["tomopel"], run, "experts up", "experts down")),
+        "closest_experts": rate(layers * 6.0 * tokens * top * ff * width, stage_ms(out["closest"], run, "experts gate_up", "experts down")),
+        "tomopel_products": rate(mixed * 2.0 * tokens * width * ((heads + 2 * kv_heads) * dim + heads + inner + channels + r_heads + heads * dim + inner)
+                                 + 2.0 * tokens * width * 4 * gru + 6.0 * tokens * width * dense_ff,
+                                 stage_ms(out["tomopel"], run, "inputs", "o", "z/x/g", "gate_up", "down")),
+        "closest_products": rate(layers * 2.0 * tokens * width * ((2 * heads + kv_heads) * dim + 4 * delta_heads * 128),
+                                 stage_ms(out["closest"], run, "q/k/v", "q/k/v/g", "o")),
+        "tomopel_streams": stream(layers * 2.0 * tokens * width * (8.0 * streams + 4 + 2), stage_ms(out["tomopel"], run, "residual add, norm")),
+        "closest_streams": stream(layers * 2.0 * tokens * width * (8.0 * streams + 4 + 2), stage_ms(out["closest_streams"], run, "residual add, norm")),
+        "tomopel_router": {"ms": round(stage_ms(out["tomopel"], run, "router"), 4)},
+        "closest_router": {"ms": round(stage_ms(out["closest"], run, "router"), 4)},
+    }
+    run = f"decode_b{batches[0]}_eager"
+    used = min(experts, batches[0] * top)          # experts a step touches at most
+    out["decode_kernels"] = {
+        "batch": batches[0], "context": context,
+        "tomopel_attention": stream(mixed * batches[0] * context * kv_heads * 2 * dim * 2.0, stage_ms(out["tomopel"], run, "attention")),
+        "closest_attention": stream(layers * batches[0] * context * kv_heads * 2 * dim * 2.0, stage_ms(out["closest"], run, "attention")),
+        "tomopel_recurrence": stream(mixed * batches[0] * inner * state * 8.0, stage_ms(out["tomopel"], run, "recurrence")),
+        "closest_recurrence": stream(layers * batches[0] * delta_heads * 128 * 128 * 8.0, stage_ms(out["closest"], run, "recurrence")),
+        "tomopel_experts": stream(routed * used * 2.0 * ff * width * 2.0, stage_ms(out["tomopel"], run, "experts up", "experts down")),
+        "closest_experts": stream(layers * used * 3.0 * ff * width * 2.0, stage_ms(out["closest"], run, "experts gate_up", "experts down")),
+        "tomopel_streams": stream(layers * 2.0 * batches[0] * width * (8.0 * streams + 4 + 2), stage_ms(out["tomopel"], run, "residual add, norm")),
+        "closest_streams": stream(layers * 2.0 * batches[0] * width * (8.0 * streams + 4 + 2), stage_ms(out["closest_streams"], run, "residual add, norm")),
+    }
+    return out
+
+
 def main() -> int:
     args = parse_args()
     world = int(os.environ.get("WORLD_SIZE", "1"))
@@ -932,6 +1077,16 @@ def main() -> int:
                 "data": "synthetic: seeded random weights, seeded uniform token ids", "sizes": args.kamedra}
         line.update(run_kamedra(args))
         line["value"] = line["kamedra"][f"decode_b8"]["tok_s"]
+        line["seconds_total"] = round(time.perf_counter() - started, 1)
+        print(json.dumps(line))
+        return 0
+
+    if args.tomopel:
+        line = {"metric": f"Tomopel at {args.tomopel} layer sizes beside the closest Rusolorn and Gizilorn models: prefill and decode",
+                "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                "data": "synthetic: seeded random weights, seeded uniform token ids", "sizes": args.tomopel}
+        line.update(run_tomopel(args))
+        line["value"] = line["tomopel"]["decode_b8"]["tok_s"]
         line["seconds_total"] = round(time.perf_counter() - started, 1)
         print(json.dumps(line))
         return 0
