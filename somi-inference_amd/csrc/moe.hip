@@ -452,7 +452,9 @@ typedef __attribute__((ext_vector_type(4))) float moe_f32x4;
 // FRAGS: row fragments of a tile (4: up to 64 rows; 1: up to 16 rows, for steps of a few tokens, where a tile is an
 // expert's one or two rows and the time is the weights' way from memory).  KS: K steps of 32 whose fragments are asked
 // for together, a round ahead (1 with four row fragments; 4 with one, so that a lane has twenty loads in flight).
-template <int MODE, int FRAGS, int KS>
+// COLF: 16-column fragments of a wavefront (4; 1, or a gate and an up fragment, where the columns alone would leave the
+// device short of workgroups).
+template <int MODE, int FRAGS, int KS, int COLF>
 __global__ void __launch_bounds__(256)
 moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16* __restrict__ w,
                         const int* __restrict__ tiles, const int* __restrict__ order,
@@ -464,7 +466,8 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
     const int first = tiles[blockIdx.x * 3 + 1], rows = tiles[blockIdx.x * 3 + 2];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int r = lane & 15, g = lane >> 4;
-    constexpr int WAVE_COLS = GATED ? 32 : 64;           // output columns of a wavefront
+    constexpr int HALF = COLF / 2;                       // GATED: as many gate fragments as up fragments
+    constexpr int WAVE_COLS = (GATED ? HALF : COLF) * 16;           // output columns of a wavefront
     const int col0 = (blockIdx.y * 4 + wave) * WAVE_COLS;
     if (col0 >= n_out) return;
     const bf16* wg = w + (int64_t)expert * (GATED ? 2 : 1) * n_out * K;
@@ -478,25 +481,25 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
         const int64_t src = alive[f] ? (GATHER ? (int64_t)(order[first + row] / top) : (int64_t)(first + row)) : 0;
         arow[f] = a + src * a_stride + g * 8;
     }
-    const bf16* brow[4];
-    bool blive[4];
+    const bf16* brow[COLF];
+    bool blive[COLF];
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-        // GATED: fragments 0, 1 are gate columns col0 .. col0 + 31, fragments 2, 3 the up rows of the same columns
-        const int col = GATED ? col0 + (c & 1) * 16 + r : col0 + c * 16 + r;
+    for (int c = 0; c < COLF; ++c) {
+        // GATED: the first half of the fragments are gate columns, the second half the up rows of the same columns
+        const int col = col0 + (GATED ? c % (HALF > 0 ? HALF : 1) : c) * 16 + r;
         blive[c] = col < n_out;
-        const int64_t wrow = GATED ? (int64_t)(c >> 1) * n_out + col : (int64_t)col;
+        const int64_t wrow = GATED && c >= HALF ? (int64_t)n_out + col : (int64_t)col;
         brow[c] = wg + (blive[c] ? wrow : 0) * K + g * 8;
     }
     const int frags = (rows + 15) >> 4;               // the same for the whole workgroup
-    moe_f32x4 acc[FRAGS][4];
+    moe_f32x4 acc[FRAGS][COLF];
 #pragma unroll
     for (int f = 0; f < FRAGS; ++f)
 #pragma unroll
-        for (int c = 0; c < 4; ++c) acc[f][c] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int c = 0; c < COLF; ++c) acc[f][c] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
     const moe_bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
-    moe_bf16x8 fa[KS][FRAGS], fb[KS][4], na[KS][FRAGS], nb[KS][4];
-    auto fetch = [&](moe_bf16x8 (&xa)[KS][FRAGS], moe_bf16x8 (&xb)[KS][4], int k0) {
+    moe_bf16x8 fa[KS][FRAGS], fb[KS][COLF], na[KS][FRAGS], nb[KS][COLF];
+    auto fetch = [&](moe_bf16x8 (&xa)[KS][FRAGS], moe_bf16x8 (&xb)[KS][COLF], int k0) {
 #pragma unroll
         for (int s = 0; s < KS; ++s) {
             const bool inside = k0 + s * 32 + g * 8 < K;
@@ -504,7 +507,7 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
             for (int f = 0; f < FRAGS; ++f)
                 xa[s][f] = (inside && alive[f]) ? *reinterpret_cast<const moe_bf16x8*>(arow[f] + k0 + s * 32) : zero;
 #pragma unroll
-            for (int c = 0; c < 4; ++c)
+            for (int c = 0; c < COLF; ++c)
                 xb[s][c] = (inside && blive[c]) ? *reinterpret_cast<const moe_bf16x8*>(brow[c] + k0 + s * 32) : zero;
         }
     };
@@ -517,7 +520,7 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
             for (int f = 0; f < FRAGS; ++f)
                 if (f < frags) {
 #pragma unroll
-                    for (int c = 0; c < 4; ++c)
+                    for (int c = 0; c < COLF; ++c)
                         acc[f][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[s][f], fb[s][c], acc[f][c], 0, 0, 0);
                 }
 #pragma unroll
@@ -525,7 +528,7 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
 #pragma unroll
             for (int f = 0; f < FRAGS; ++f) fa[s][f] = na[s][f];
 #pragma unroll
-            for (int c = 0; c < 4; ++c) fb[s][c] = nb[s][c];
+            for (int c = 0; c < COLF; ++c) fb[s][c] = nb[s][c];
         }
     }
     // a lane holds rows g * 4 + i of a fragment's 16 and column r of its 16
@@ -539,15 +542,15 @@ moe_product_mfma_kernel(const bf16* __restrict__ a, int64_t a_stride, const bf16
             const float pw = pair_weight != nullptr ? pair_weight[pair] : 1.0f;
             if (GATED) {
 #pragma unroll
-                for (int c = 0; c < 2; ++c) {
+                for (int c = 0; c < HALF; ++c) {
                     const int col = col0 + c * 16 + r;
                     if (col < n_out)
                         ((bf16*)out_)[(int64_t)(first + row) * n_out + col] =
-                            (bf16)clamped_glu(pw * acc[f][c][i], pw * acc[f][c + 2][i], limit, alpha, shift);
+                            (bf16)clamped_glu(pw * acc[f][c][i], pw * acc[f][c + HALF][i], limit, alpha, shift);
                 }
             } else {
 #pragma unroll
-                for (int c = 0; c < 4; ++c) {
+                for (int c = 0; c < COLF; ++c) {
                     const int col = col0 + c * 16 + r;
                     if (col >= n_out) continue;
                     if (MODE == MOE_SQUARED_RELU) ((bf16*)out_)[(int64_t)(first + row) * n_out + col] = (bf16)squared_relu(pw * acc[f][c][i]);
@@ -700,8 +703,12 @@ extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void
                  "moe_product_mfma: K of %d or rows that are not aligned to 16 bytes", K);
     SOMI_REQUIRE(mode == MOE_DOWN || mode == MOE_GATED || mode == MOE_SQUARED_RELU, "moe_product_mfma: unknown mode %d", mode);
     if (max_tiles == 0) return 0;
-    const int wide = tile_rows == MOE_BIG_ROWS ? 1 : 2;              // columns of a workgroup: 64 or 128 gated, else twice that
-    const dim3 grid(max_tiles, ceil_div(n_out, (mode == MOE_GATED ? 64 : 128) * wide));
+    // columns of a workgroup: 64 gated in the large tiles and 128 in the others, twice that without a gate; for steps of a
+    // few tokens a quarter where that alone would be less than two workgroups a compute unit (a row's sums are the same)
+    int cols = (mode == MOE_GATED ? 64 : 128) * (tile_rows == MOE_BIG_ROWS ? 1 : 2);
+    const bool narrow = tile_rows == 16 && (int64_t)max_tiles * ceil_div(n_out, cols) < 2 * (int64_t)somi_units();
+    if (narrow) cols = 64;
+    const dim3 grid(max_tiles, ceil_div(n_out, cols));
     SOMI_REQUIRE(grid.y <= 65535, "moe_product_mfma: too many columns");
 #define MOE_LAUNCH(...)                                                                                                   \
     hipLaunchKernelGGL((__VA_ARGS__), grid, dim3(256), 0, stream, (const bf16*)a, a_stride, (const bf16*)w, tiles, order, \
@@ -709,8 +716,9 @@ extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void
 #define MOE_BY_ROWS(MODE)                                                                             \
     do {                                                                                              \
         if (tile_rows == MOE_BIG_ROWS) MOE_LAUNCH(moe_product_tile_kernel<MODE>);                     \
-        else if (tile_rows == 16) MOE_LAUNCH(moe_product_mfma_kernel<MODE, 1, 4>);                    \
-        else MOE_LAUNCH(moe_product_mfma_kernel<MODE, MOE_MFMA_FRAGS, 1>);                            \
+        else if (narrow) MOE_LAUNCH(moe_product_mfma_kernel<MODE, 1, 8, (MODE == MOE_GATED ? 2 : 1)>); \
+        else if (tile_rows == 16) MOE_LAUNCH(moe_product_mfma_kernel<MODE, 1, 4, 4>);                 \
+        else MOE_LAUNCH(moe_product_mfma_kernel<MODE, MOE_MFMA_FRAGS, 1, 4>);                         \
     } while (0)
     if (mode == MOE_GATED) MOE_BY_ROWS(MOE_GATED);
     else if (mode == MOE_DOWN) MOE_BY_ROWS(MOE_DOWN);

@@ -1774,11 +1774,17 @@ def _float_rows(t: torch.Tensor, n: int, width: int, name: str) -> ctypes.c_int6
     return ctypes.c_int64(t.stride(0))
 
 
-def ssd_scan(xbc: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor,
-             entry_start: torch.Tensor, state_slots: torch.Tensor, state: torch.Tensor, groups: int) -> torch.Tensor:
+def ssd_chunked(p: int, n_state: int) -> bool:
+    """The chunked kernels take heads of ``p`` channels with a state of ``n_state`` rows."""
+    return bool(library().somi_ssd_chunked(int(p), int(n_state)))
+
+
+def ssd(xbc: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor, step,
+        state: torch.Tensor, groups: int, chunked: bool = True) -> torch.Tensor:
     """S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + D x per head with dt = softplus(raw + dt_bias) -> y [N, heads * P]
     float32.  xbc: [N, heads * P + 2 groups * N_state] float32, x then B then C; raw_dt: [N, heads] float32, possibly
-    columns of wider rows; state: [slots, heads, P, N_state] float32, read and written in place."""
+    columns of wider rows; state: [slots, heads, P, N_state] float32, read and written in place.  ``chunked``: entries long
+    enough go through matrix products chunk by chunk where the sizes allow; else every entry is walked token by token."""
     _need(state, "recurrent state", torch.float32)
     _, heads, p, n_state = state.shape
     n = xbc.shape[0]
@@ -1786,12 +1792,18 @@ def ssd_scan(xbc: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, a_l
     stride = _float_rows(raw_dt, n, heads, "dt rows")
     for t, name in ((dt_bias, "dt bias"), (a_log, "decay rates"), (skip, "skip weights")):
         _need(t, name, torch.float32, (heads,))
-    entries = state_slots.numel()
-    _need(entry_start, "entry offsets", torch.int32, (entries + 1,))
-    _need(state_slots, "state slots", torch.int32, (entries,))
+    entries = step.state_slots.numel()
+    _need(step.entry_start, "entry offsets", torch.int32, (entries + 1,))
+    _need(step.state_slots, "state slots", torch.int32, (entries,))
     y = torch.empty((n, heads * p), dtype=torch.float32, device=xbc.device)
-    _check(library().somi_ssd_scan(_ptr(xbc), _ptr(raw_dt), stride, _ptr(dt_bias), _ptr(a_log), _ptr(skip), _ptr(entry_start),
-                                   _ptr(state_slots), _ptr(state), entries, heads, int(groups), p, n_state, _ptr(y), _stream()))
+    local = decay = None
+    if chunked and step.max_entry_len >= library().somi_ssd_chunked_from() and ssd_chunked(p, n_state):
+        chunks = library().somi_ssd_chunks(n, entries)
+        local = torch.empty((chunks, heads, p, n_state), dtype=torch.float32, device=xbc.device)
+        decay = torch.empty((chunks, heads), dtype=torch.float32, device=xbc.device)
+    _check(library().somi_ssd(_ptr(xbc), _ptr(raw_dt), stride, _ptr(dt_bias), _ptr(a_log), _ptr(skip), _ptr(step.entry_start),
+                              _ptr(step.state_slots), _ptr(state), entries, int(step.max_entry_len), heads, int(groups), p,
+                              n_state, _ptr(local), _ptr(decay), _ptr(y), _stream()))
     return y
 
 

@@ -103,7 +103,6 @@ class Mamba2(RowsMixer):
         with stage("convolution"):
             xbc = ops.conv_silu(xbc, self.conv_taps, self.conv_bias, conv, step)
         with stage("recurrence"):
-            y = ops.ssd_scan(xbc, dt, self.dt_bias, self.a_log, self.skip, step.entry_start, step.state_slots, state,
-                             self.num_groups)
+            y = ops.ssd(xbc, dt, self.dt_bias, self.a_log, self.skip, step, state, self.num_groups)
         with stage("gate, norm"):
             ops.gated_group_norm(y, z, self.norm_weight, self.norm_groups, self.eps, scale, out)

@@ -239,7 +239,7 @@ def mamba_part(heads, vdim, state, groups, taps, norm_groups, hidden=48):
 
 MAMBA = [  # heads, vdim, state, groups, taps, normed parts
     (4, 16, 16, 2, 4, 2), (3, 10, 5, 1, 1, 1), (2, 24, 33, 2, 2, 3), (6, 7, 64, 3, 3, 6), (2, 40, 130, 1, 4, 1),
-    (1, 66, 31, 1, 9, 2), (4, 8, 200, 2, 5, 4), (2, 5, 300, 1, 4, 1),
+    (1, 66, 31, 1, 9, 2), (4, 8, 200, 2, 5, 4), (2, 5, 300, 1, 4, 1), (2, 64, 128, 1, 4, 1), (3, 20, 48, 3, 4, 2),
 ]
 
 
@@ -275,6 +275,55 @@ def test_mamba2_whole_cut_and_side_by_side(dtype, sizes):
     check(torch.cat(got_a), want, dtype)
     done = torch.cat(got_b)
     check(done, want_other[:done.shape[0]], dtype)
+
+
+def step_of(lengths):
+    """What the recurrence reads of a step with entries of these lengths, in slots that are not in order."""
+    from types import SimpleNamespace
+    starts = [0]
+    for n in lengths:
+        starts.append(starts[-1] + n)
+    slots = [(3 * i + 1) % (3 * len(lengths)) for i in range(len(lengths))]
+    return SimpleNamespace(entry_start=torch.tensor(starts, dtype=torch.int32, device=DEV), max_entry_len=max(lengths),
+                           state_slots=torch.tensor(slots, dtype=torch.int32, device=DEV)), starts, slots
+
+
+@pytest.mark.parametrize("heads,p,n_state,groups", [(2, 64, 128, 1), (4, 16, 16, 2), (3, 12, 20, 3), (2, 100, 36, 1), (1, 132, 256, 1), (6, 8, 4, 2)])
+@pytest.mark.parametrize("lengths", [[64], [65], [127, 1, 128], [3, 200, 63, 64, 1, 333]])
+def test_the_recurrence_in_chunks_is_the_recurrence_token_by_token(heads, p, n_state, groups, lengths):
+    """Both forms from the same states, against each other and against the plain function in float64; decays from almost
+    one to almost zero stand side by side in a chunk."""
+    gen = torch.Generator().manual_seed(heads * p + len(lengths))
+    step, starts, slots = step_of(lengths)
+    n, total = starts[-1], heads * p + 2 * groups * n_state
+    xbc, rows = torch.randn(n, total, generator=gen), torch.randn(n, heads + 3, generator=gen) * 3
+    bias, a_log, skip = (torch.randn(heads, generator=gen) * s for s in (2.0, 1.5, 1.0))
+    state = torch.randn(3 * len(lengths), heads, p, n_state, generator=gen)
+    assert ops.ssd_chunked(p, n_state)
+    got = {}
+    for chunked in (True, False):
+        kept = state.to(DEV)
+        y = ops.ssd(xbc.to(DEV), rows.to(DEV)[:, 3:], bias.to(DEV), a_log.to(DEV), skip.to(DEV), step, kept, groups, chunked=chunked)
+        got[chunked] = (y.cpu(), kept.cpu())
+    for e, length in enumerate(lengths):
+        at = slice(starts[e], starts[e] + length)
+        x, b, c = torch.split(xbc[at].double(), [heads * p, groups * n_state, groups * n_state], dim=1)
+        dt = plain.softplus(rows[at, 3:].double() + bias.double())
+        b, c = b.view(length, groups, -1).repeat_interleave(heads // groups, 1), c.view(length, groups, -1).repeat_interleave(heads // groups, 1)
+        s, want = state[slots[e]].double(), []
+        for t in range(length):
+            s = torch.exp(-torch.exp(a_log.double()) * dt[t])[:, None, None] * s + (dt[t][:, None] * x[t].view(heads, p))[:, :, None] * b[t][:, None, :]
+            want.append((s * c[t][:, None, :]).sum(-1) + skip.double()[:, None] * x[t].view(heads, p))
+        want = torch.stack(want).view(length, -1).float()
+        for chunked in (True, False):
+            torch.testing.assert_close(got[chunked][0][at], want, rtol=1e-4, atol=2e-5 * float(want.abs().max()))
+            torch.testing.assert_close(got[chunked][1][slots[e]], s.float(), rtol=1e-4, atol=2e-5 * float(s.abs().max()))
+    idle = [i for i in range(3 * len(lengths)) if i not in slots]
+    assert all(torch.equal(got[chunked][1][idle], state[idle]) for chunked in (True, False))
+
+
+def test_which_sizes_the_chunked_recurrence_takes():
+    assert not ops.ssd_chunked(10, 16) and not ops.ssd_chunked(16, 33) and not ops.ssd_chunked(16, 300)
 
 
 def test_the_state_remembers_and_the_next_request_starts_from_zero():
