@@ -317,11 +317,12 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
         const int page_lo = (begin & ~31) >> shift, page_last = end >> shift;
         const int page_count = ((end | 31) >> shift) - page_lo + 1;
         for (int i = tid; i < page_count; i += 256) pages[i] = table[min(page_lo + i, page_last)];
-        // the bias of this split's keys: only a split that reaches the token's nearest keys has any
+        // the bias of this split's keys: only a split whose 32-key tiles (the last one reaches past the split's keys) come
+        // near the token has any
         const float inv_scale = 1.0f / scale;
         const int bias_rows = G < 16 ? G : 16;
         const int bias_row = r < bias_rows ? r : bias_rows - 1;
-        if (BIAS && bias.in_lds && p - end < bias.length) {
+        if (BIAS && bias.in_lds && p - (end | 31) < bias.length) {
             for (int i = tid; i < bias_rows * bias.length; i += 256) {
                 const int hl = hb * 16 + i / bias.length;
                 bias_s[i] = bias.table[(int64_t)(kvh * G + (hl < G ? hl : G - 1)) * bias.length + i % bias.length] * inv_scale;

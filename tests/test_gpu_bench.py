@@ -192,3 +192,29 @@ def test_gizilorn_option_runs_the_models_and_leaves_the_default_alone():
     assert "mixed attention" in line["gizilorn"]["stages"]["prefill_512"] and line["value"] == line["gizilorn"]["decode_b8"]["tok_s"]
     assert line["prefill_kernels"]["gizilorn_attention"]["ms"] > 0 and line["decode_kernels"]["gizilorn_latent_attention"]["ms"] > 0
     assert line["prefill_kernels"]["gizilorn_streams"]["gbs"] > 0
+
+
+def test_tomopel_option_runs_the_models_and_leaves_the_default_alone():
+    """``--tomopel`` runs a Tomopel model beside the closest Rusolorn and Gizilorn models and prints one JSON line; the
+    sizes' config.json dicts are what the registry takes."""
+    import bench
+    from somi_inference_amd.config import config_from_dict
+    for sizes in bench.TOMOPEL_SIZES:
+        arch, config = config_from_dict(bench.tomopel_config_dict(sizes))
+        assert arch.name == "Tomopel" and len(config.layers) == bench.TOMOPEL_LAYERS and config.streams == 2
+        assert [layer.type for layer in config.layers].count("parallel") == bench.TOMOPEL_PARALLEL
+        arch, closest = config_from_dict(bench.tomopel_closest_config_dict(sizes))
+        right, theirs = config.layers[0].mixer.right, closest.layers[0].right
+        assert arch.name == "Rusolorn" and closest.width == config.width
+        assert theirs.heads * theirs.dim * theirs.vdim == right.heads * right.vdim * right.state
+        arch, closest = config_from_dict(bench.tomopel_closest_streams_config_dict(sizes))
+        assert arch.name == "Gizilorn" and closest.width == config.width and closest.streams == config.streams
+    done = subprocess.run([sys.executable, os.path.join(ROOT, "bench.py"), "--tomopel", "1b", "--steps", "16", "--warmup", "2",
+                           "--prefill-tokens", "512", "--context", "1024"], capture_output=True, text=True, timeout=900, cwd=ROOT)
+    assert done.returncode == 0, done.stderr[-3000:]
+    line = json.loads([row for row in done.stdout.splitlines() if row.startswith("{")][-1])
+    for model in ("tomopel", "closest", "closest_streams"):
+        assert line[model]["decode_b8"]["tok_s"] > 0 and line[model]["prefill"]["512"]["value"] > 0
+    assert {"attention", "recurrence", "gated recurrence", "experts up"} <= set(line["tomopel"]["stages"]["prefill_512"])
+    assert line["value"] == line["tomopel"]["decode_b8"]["tok_s"]
+    assert line["prefill_kernels"]["tomopel_recurrence"]["ms"] > 0 and line["decode_kernels"]["tomopel_attention"]["ms"] > 0

@@ -216,6 +216,28 @@ def test_every_launch_shape_of_the_prompt_kernels_with_a_bias(dim, shape, length
         check(out, want, torch.bfloat16)
 
 
+@pytest.mark.parametrize("dim", [32, 64, 128])
+@pytest.mark.parametrize("length", [2, 9, 21, 40])
+def test_a_split_that_ends_just_beyond_the_bias_reads_no_leftover_of_another_launch(dim, length):
+    """A split's last 32-key tile reaches past its keys and may come near enough for the bias though none of its keys
+    does.  Before every launch another one, whose table is not a number anywhere, leaves its table in LDS."""
+    gen = torch.Generator().manual_seed(dim + length)
+    n, nq, nkv = 260, 4, 2
+    kc, vc, table = paged(n, nkv, dim, 8, gen)
+    q = torch.randn(n, nq * dim, generator=gen).to(torch.bfloat16).to(DEV)
+    bias = torch.randn(nq, length, generator=gen) * 3
+    bias[:, -1] = 0.0
+    bias = bias.to(DEV)
+    poison = torch.full((nq, 600), float("nan"), device=DEV)
+    positions, entry = torch.arange(n, dtype=torch.int32, device=DEV), torch.zeros(n, dtype=torch.int32, device=DEV)
+    want = ops.paged_attention_plain(q, q.shape[1], kc, vc, table, entry, positions, nq, 0, 0.2, bias)
+    for split_len, splits in ((64, 5), (272, 1), (144, 2), (96, 3)):
+        out, waste = torch.empty_like(want), torch.empty_like(want)
+        ops.attention_decode(q, q.shape[1], kc, vc, table, entry, positions, nq, 0, 0.2, split_len, splits, waste, bias=poison)
+        ops.attention_decode(q, q.shape[1], kc, vc, table, entry, positions, nq, 0, 0.2, split_len, splits, out, bias=bias)
+        check(out, want, torch.bfloat16)
+
+
 def test_sizes_without_a_matrix_core_kernel_for_the_bias_are_refused_by_it():
     gen = torch.Generator().manual_seed(1)
     kc, vc, table = paged(20, 1, 144, 8, gen)
