@@ -8,12 +8,10 @@
 // A step of S is the map s -> a s + b with a = 1 - z, b = z c, and maps compose: a workgroup owns GRU_CH channels of one
 // entry and walks its tokens SEGS * GRU_T at a time; thread (segment, channel) composes the maps of its GRU_T tokens, the
 // segments' maps meet in LDS, each thread runs the state through the segments before its own and then through its tokens.
-// SEGS is 1 in steps of few tokens an entry.
+// SEGS is 1 in steps of few tokens an entry, which run 64 channels a workgroup; else 16.
 #include "common.h"
 
-#define GRU_CH 32
-
-template <typename T, int SEGS, int GRU_T>
+template <typename T, int GRU_CH, int SEGS, int GRU_T>
 __global__ void __launch_bounds__(GRU_CH * SEGS)
 min_gru_kernel(const float* __restrict__ rows, int64_t row_stride, const float* __restrict__ bz, const float* __restrict__ bx,
                const int* __restrict__ entry_start, const int* __restrict__ state_slots, float* __restrict__ state, int width,
@@ -77,19 +75,21 @@ extern "C" int somi_min_gru(const float* rows, int64_t row_stride, const float* 
                             void* out, int64_t out_stride, int dtype, hipStream_t stream) {
     SOMI_REQUIRE(n_entries >= 0 && max_entry_len >= 0 && width > 0 && row_stride >= 3 * (int64_t)width && out_stride >= width,
                  "min_gru: bad sizes");
-    SOMI_REQUIRE(ceil_div(width, GRU_CH) <= 65535, "min_gru: too many channels");
+    SOMI_REQUIRE(ceil_div(width, 16) <= 65535, "min_gru: too many channels");
     if (n_entries == 0) return 0;
-    const dim3 grid(n_entries, ceil_div(width, GRU_CH));
-#define SOMI_GRU(T, SEGS, TOKENS)                                                                                          \
-    hipLaunchKernelGGL((min_gru_kernel<T, SEGS, TOKENS>), grid, dim3(GRU_CH * SEGS), 0, stream, rows, row_stride, bz, bx,  \
-                       entry_start, state_slots, state, width, scale, (T*)out, out_stride)
-    if (dtype == SOMI_F32) {
-        if (max_entry_len == 1) SOMI_GRU(float, 1, 1); else if (max_entry_len <= 16) SOMI_GRU(float, 1, 4); else SOMI_GRU(float, 32, 8);
-    } else if (dtype == SOMI_BF16) {
-        if (max_entry_len == 1) SOMI_GRU(bf16, 1, 1); else if (max_entry_len <= 16) SOMI_GRU(bf16, 1, 4); else SOMI_GRU(bf16, 32, 8);
-    } else {
-        return somi_fail("min_gru: unknown dtype %d", dtype);
-    }
+#define SOMI_GRU(T, CH, SEGS, TOKENS)                                                                                       \
+    hipLaunchKernelGGL((min_gru_kernel<T, CH, SEGS, TOKENS>), dim3(n_entries, ceil_div(width, CH)), dim3(CH * SEGS), 0,     \
+                       stream, rows, row_stride, bz, bx, entry_start, state_slots, state, width, scale, (T*)out, out_stride)
+#define SOMI_GRU_BY_LENGTH(T)                              \
+    do {                                                   \
+        if (max_entry_len == 1) SOMI_GRU(T, 64, 1, 1);     \
+        else if (max_entry_len <= 16) SOMI_GRU(T, 64, 1, 4); \
+        else SOMI_GRU(T, 16, 64, 8);                       \
+    } while (0)
+    if (dtype == SOMI_F32) SOMI_GRU_BY_LENGTH(float);
+    else if (dtype == SOMI_BF16) SOMI_GRU_BY_LENGTH(bf16);
+    else return somi_fail("min_gru: unknown dtype %d", dtype);
+#undef SOMI_GRU_BY_LENGTH
 #undef SOMI_GRU
     SOMI_LAUNCH_CHECK("min_gru");
     return 0;

@@ -446,8 +446,10 @@ gated_group_norm_kernel(const float* __restrict__ y, const float* __restrict__ z
     };
 #pragma unroll
     for (int j = 0; j < HELD; ++j) {
+        if (256 * j >= part) break;                      // the same for the whole workgroup
         const int c = threadIdx.x + 256 * j;
-        held[j] = c < part ? value(c) : 0.f;
+        const float v = value(min(c, part - 1));
+        held[j] = c < part ? v : 0.f;
         ss = fmaf(held[j], held[j], ss);
     }
     for (int c = threadIdx.x + 256 * HELD; c < part; c += 256) {
