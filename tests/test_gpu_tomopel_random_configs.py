@@ -2,7 +2,8 @@
 key/value heads, value sizes unlike key sizes, tables of few and many buckets, bias reaches shorter and longer than the
 sequences, temperatures or none, groups, normed parts and taps of the recurrence, minGRU widths, dense and routed
 feed-forwards or none, widths that are no multiple of 8, page sizes) under random mixed traces with so few pages that they
-are used again: the engine against the plain implementation and against itself on the whole prompt."""
+are used again: the engine against the plain implementation and against itself on the whole prompt.  Pages, states and
+the memory the engine allocates from hold values that are not numbers before it starts."""
 
 import random
 
@@ -53,6 +54,16 @@ def random_config(rng: random.Random) -> TomopelConfig:
                          residual_mult=rng.choice([1.0, 0.3, 0.7]), streams=rng.choice([None, 1, 2, 3, 4, 8]), layers=tuple(layers))
 
 
+def leave_no_zeros(runner) -> None:
+    """Whatever is read before it is written shows: the cache's tensors and freed device memory become not a number."""
+    for cache in runner.cache.layer_caches:
+        for leaf in cache.leaves():
+            for tensor in list(leaf.tensors.values()) + ([leaf.state] if leaf.state is not None else []):
+                tensor.fill_(float("nan"))
+    held = [torch.full((size,), float("nan"), device="cuda:0") for size in (1 << 22, 1 << 18, 1 << 14, 1 << 10, 100) for _ in range(8)]
+    del held
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("seed", range(24))
 def test_random_configuration_under_a_random_mixed_trace(seed, dtype, tmp_path):
@@ -71,6 +82,7 @@ def test_random_configuration_under_a_random_mixed_trace(seed, dtype, tmp_path):
     steps = mixed_trace(requests, seed=rng.randrange(1000), portion_sizes=sizes)
     pages = peak_pages(steps, block_size)
     runner, _ = make_engine(folder, dtype, block_size, pages, max_requests=4)
+    leave_no_zeros(runner)
     rows = {rid: [] for rid in requests}
     for entries, ends in steps:
         batch = []
