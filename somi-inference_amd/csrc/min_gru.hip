@@ -8,7 +8,7 @@
 // A step of S is the map s -> a s + b with a = 1 - z, b = z c, and maps compose: a workgroup owns GRU_CH channels of one
 // entry and walks its tokens SEGS * GRU_T at a time; thread (segment, channel) composes the maps of its GRU_T tokens, the
 // segments' maps meet in LDS, each thread runs the state through the segments before its own and then through its tokens.
-// SEGS is 1 in steps of few tokens an entry, which run 64 channels a workgroup; else 16.
+// SEGS is 1 in steps of few tokens an entry, which run 64 channels a workgroup; else 64, with 16 channels.
 #include "common.h"
 
 template <typename T, int GRU_CH, int SEGS, int GRU_T>
