@@ -1,4 +1,4 @@
-// A gated recurrence whose gates read only the current token (minGRU), element by element:
+// minGRU, a recurrence whose gate does not look at its state, element by element:
 //
 //     z = sigmoid(rz + b_z),   u = rx + b_x,   c = u + 1/2 for u >= 0 and sigmoid(u) for u < 0
 //     S_t = (1 - z) S_(t-1) + z c;     out = scale * S_t * silu(rg)
@@ -8,7 +8,8 @@
 // A step of S is the map s -> a s + b with a = 1 - z, b = z c, and maps compose: a workgroup owns GRU_CH channels of one
 // entry and walks its tokens SEGS * GRU_T at a time; thread (segment, channel) composes the maps of its GRU_T tokens, the
 // segments' maps meet in LDS, each thread runs the state through the segments before its own and then through its tokens.
-// SEGS is 1 in steps of few tokens an entry, which run 64 channels a workgroup; else 64, with 16 channels.
+// SEGS is 1 in steps of few tokens an entry, which run 64 channels a workgroup; else 64, with 16 channels, where an entry
+// that fits one segment (a decoded token beside a prompt's portion) leaves the other segments and the meeting out.
 #include "common.h"
 
 template <typename T, int GRU_CH, int SEGS, int GRU_T>
@@ -22,6 +23,8 @@ min_gru_kernel(const float* __restrict__ rows, int64_t row_stride, const float* 
     const bool live = c < width;
     const int cc = live ? c : width - 1;
     const int t0 = entry_start[e], t1 = entry_start[e + 1];
+    const bool alone = SEGS == 1 || t1 - t0 <= GRU_T;             // the same for the whole workgroup
+    if (alone && seg > 0) return;
     float* kept = state + (int64_t)state_slots[e] * width + cc;
     float s = *kept;
     const float wz = bz[cc], wx = bx[cc];
@@ -48,7 +51,7 @@ min_gru_kernel(const float* __restrict__ rows, int64_t row_stride, const float* 
             cb = fmaf(a[i], cb, b[i]);
         }
         float mine = s;
-        if (SEGS > 1) {
+        if (!alone) {
             __syncthreads();                     // the last round's maps are read
             map_a[seg][ch] = ca;
             map_b[seg][ch] = cb;
@@ -64,7 +67,7 @@ min_gru_kernel(const float* __restrict__ rows, int64_t row_stride, const float* 
             if (live && first + i < t1)
                 out[(int64_t)(first + i) * out_stride + c] = from_float<T>(scale * mine * (gate[i] / (1.0f + expf(-gate[i]))));
         }
-        if (SEGS == 1) s = mine;
+        if (alone) s = mine;
     }
     if (live && seg == 0) *kept = s;
 }

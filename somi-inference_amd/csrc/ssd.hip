@@ -425,9 +425,9 @@ extern "C" int somi_ssd(const float* xbc, const float* raw, int64_t raw_stride, 
 }
 
 // ------------------------------------------------------------------------------------------------ gate and norm
-// u = y * silu(z), each of `groups` equal parts of a row divided by its own root mean square (eps inside the root), times
-// w and `scale`.  A workgroup a (token, part).  y: [n, width] float32; z: float32, rows z_stride apart; out: rows of
-// `width`, out_stride apart.
+// u = y * silu(z), RMS-normed in `groups` equal parts of a row (eps inside the root), times w and `scale`.  A
+// workgroup a (token, part).  y: [n, width] float32; z: float32, rows z_stride apart; out: rows of `width`, out_stride
+// apart.
 template <typename T>
 __global__ void __launch_bounds__(256)
 gated_group_norm_kernel(const float* __restrict__ y, const float* __restrict__ z, int64_t z_stride,

@@ -1809,8 +1809,8 @@ def ssd(xbc: torch.Tensor, raw_dt: torch.Tensor, dt_bias: torch.Tensor, a_log: t
 
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, scale: float,
                      out: torch.Tensor) -> None:
-    """out = scale * weight * (y silu(z)), each of ``groups`` equal parts of a row divided by its own root mean square.  y:
-    [N, width] float32; z: float32, possibly columns of wider rows; out: [N, width], likewise."""
+    """out = scale * weight * (y silu(z)), RMS-normed in ``groups`` equal parts of a row.  y: [N, width] float32; z:
+    float32, possibly columns of wider rows; out: [N, width], likewise."""
     _need(y, "rows", torch.float32)
     n, width = y.shape
     _need(weight, "norm weight", torch.float32, (width,))

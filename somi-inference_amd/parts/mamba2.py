@@ -1,17 +1,17 @@
 """Mamba-2 (state-space duality): a recurrent mixer whose decay is one number a head and token.
 
 One product of the input gives ``z | x | B | C | dt`` (inner = heads * value_dim channels of z and of x, ``groups *
-state_dim`` of B and of C, one dt a head).  x, B and C together pass a short causal convolution with a bias and SiLU
-(the last tap on the current token, zeros before the start); then, head by head (head h reads group ``h // (heads /
-groups)`` of B and C),
+state_dim`` of B and of C, one dt a head).  A short causal convolution with a bias and SiLU runs over the channels of x, B
+and C (zeros stand before a request's first token, the last tap meets the token itself); then, head by head (head h reads
+group ``h // (heads / groups)`` of B and C),
 
     dt  = softplus(dt + dt_bias)
     S   = exp(-exp(A_log) dt) S + dt B x^T;      y = S^T C + D x              (S: state_dim x value_dim, from zero)
 
-y (the heads side by side) times ``silu(z)`` is divided by its root mean square in ``norm_groups`` equal parts, times a
-weight, and projected by W_o.  A request's S and the convolution's last ``taps - 1`` inputs live in float32 in its state
-slot and are carried from step to step; the convolution, dt, the decay, the recurrence, the gate and the norm are float32
-in both engines.
+y (the heads side by side) times ``silu(z)`` is cut into ``norm_groups`` equal parts, each part RMS-normed, the whole
+times a weight, and projected by W_o.  A request's S and the ``taps - 1`` newest inputs of the convolution live in float32
+in its state slot and are carried from step to step; the convolution, dt, the decay, the recurrence, the gate and the norm
+are float32 in both engines.
 """
 
 from __future__ import annotations

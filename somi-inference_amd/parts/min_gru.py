@@ -1,4 +1,4 @@
-"""minGRU: a gated recurrence whose gates read only the current token.
+"""minGRU: a recurrence whose update gate and candidate do not look at its state.
 
     z = sigmoid(W_z h + b_z),   u = W_x h + b_x,   c = u + 1/2 where u >= 0 and sigmoid(u) where u < 0
     S <- (1 - z) S + z c                              (element by element, from zero)

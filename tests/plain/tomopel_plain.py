@@ -117,7 +117,7 @@ def ssd(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, dt: torch.Tensor, a_l
 
 
 def grouped_rms(y: torch.Tensor, groups: int, eps: float) -> torch.Tensor:
-    """Each of ``groups`` equal parts of a row divided by its own root mean square."""
+    """A row's ``groups`` equal parts, RMS-normed one by one."""
     T = y.shape[0]
     return rms(y.view(T, groups, -1), eps).reshape(T, -1)
 

@@ -409,13 +409,17 @@ def test_min_gru_whole_cut_and_side_by_side(dtype, width):
         check(cut, want, dtype)
         if dtype == torch.float32:
             torch.testing.assert_close(cut, whole, rtol=2e-5, atol=2e-5)
-    got_a, got_b = [], []
-    for i in range(30):                      # single tokens of one request beside portions of the other
-        outs = engine.run([("a", x[11 * i:11 * i + 11]), ("b", other[i:i + 1])])[0]
-        got_a.append(outs[0])
-        got_b.append(outs[1])
-    check(torch.cat(got_a), want, dtype)
-    check(torch.cat(got_b), want_other, dtype)
+    for size, small in ((11, [1] * 30), (33, [1, 8, 9, 1, 2, 1, 1, 1, 1, 5])):
+        got_a, got_b, at = [], [], 0
+        for i, few in enumerate(small):      # few tokens of one request beside portions of the other
+            outs = engine.run([("a", x[size * i:size * i + size]), ("b", other[at:at + few])])[0]
+            at += few
+            got_a.append(outs[0])
+            got_b.append(outs[1])
+        check(torch.cat(got_a), want, dtype)
+        check(torch.cat(got_b), want_other, dtype)
+        for rid in ("a", "b"):
+            engine.cache.free(rid)
 
 
 def test_min_gru_gates_far_out_and_the_candidate_on_both_sides_of_zero():
