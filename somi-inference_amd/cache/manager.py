@@ -9,11 +9,12 @@ duplicate ``register_sequence`` raises "already registered" (:150-156).
 
 Beyond the reference: a layer says what it keeps per token (a ``PagedSpec``: the
 tensors of a page, a window, a page size of its own if its kernels want one) and
-layers are put into *groups* by window (with the first tokens it keeps) and page size.  The layers of a group
+layers are put into *groups* by window (with the first tokens it keeps), chunk and page size.  The layers of a group
 share one page pool and one block table per request; each has tensors of its own,
 allocated as its spec lists them.  A group with a window releases a page as soon
 as the window has passed it, while the request is still live, unless the page
-holds some of the request's first tokens that the window keeps visible.  Every group's pool
+holds some of the request's first tokens that the window keeps visible; one with chunks
+as soon as the next token belongs to a later chunk than all of the page's.  Every group's pool
 holds the same number of tokens, ``num_blocks * block_size``, cut into pages of
 the group's size.  Mixers with fixed-size state get one slot per request in a
 state tensor, zeroed when the request is registered.
@@ -40,6 +41,12 @@ class PagedGroup:
     page_size: int = 0
     keep_first: int = 0                                  # a request's first tokens that stay beside the window
     runs: list[int] = field(default_factory=list)      # layer runs whose tensors use this group's page ids
+    chunk: int | None = None                             # a token sees only its own run of this many positions
+
+    def first_visible(self, position: int) -> int:
+        """The first position that a token at ``position`` sees, kept first tokens aside."""
+        first = 0 if self.window is None else max(0, position - self.window + 1)
+        return first if self.chunk is None else max(first, position // self.chunk * self.chunk)
 
 
 @dataclass
@@ -73,7 +80,7 @@ class CacheManager:
         self.dtype, self.device = dtype, torch.device(device)
         self.groups: list[PagedGroup] = []
         self.layer_caches: list[LayerCache | None] = [None] * len(needs)
-        self._by_need: dict[tuple[int | None, int, int], int] = {}
+        self._by_need: dict[tuple[int | None, int, int, int | None], int] = {}
         self._allocate = bool(allocate_tensors)
         self._borrowed: list[tuple[LayerCache, str, BorrowedCache, int]] = []
         for run, need in enumerate(needs):
@@ -119,13 +126,13 @@ class CacheManager:
         if isinstance(need, PagedSpec):
             page_size = int(need.page_size or self.block_size)
             keep_first = int(need.keep_first) if need.window is not None else 0
-            key = (need.window, page_size, keep_first)
+            key = (need.window, page_size, keep_first, need.chunk)
             if key not in self._by_need:
                 pages = self.pool_tokens // page_size
                 if pages < 1:
                     raise ValueError(f"a pool of {self.pool_tokens} tokens holds no page of {page_size}")
                 self._by_need[key] = len(self.groups)
-                self.groups.append(PagedGroup(need.window, PagePool(pages), page_size, keep_first))
+                self.groups.append(PagedGroup(need.window, PagePool(pages), page_size, keep_first, chunk=need.chunk))
             group = self._by_need[key]
             self.groups[group].runs.append(run)
             tensors = {}
@@ -264,14 +271,13 @@ class CacheManager:
         for g, (group, pages) in enumerate(zip(self.groups, record.pages)):
             if self._pages_for(group, record.num_tokens) > len(pages):
                 raise CacheError(f"request {request_id!r}: tokens committed beyond the reserved pages")
-            if group.window is None:
+            if group.window is None and group.chunk is None:
                 continue
-            # The next token sits at position num_tokens and sees keys from
-            # num_tokens - window + 1 on; pages wholly below that are done, but for
-            # the pages that hold any of the request's kept first tokens.
-            first_visible = record.num_tokens - group.window + 1
+            # The next token sits at position num_tokens; pages wholly below what it sees
+            # are done, but for the pages that hold any of the request's kept first tokens.
+            first_visible = group.first_visible(record.num_tokens)
             kept_pages = self._pages_for(group, group.keep_first)
-            for logical in range(kept_pages, min(len(pages), max(0, first_visible) // group.page_size)):
+            for logical in range(kept_pages, min(len(pages), first_visible // group.page_size)):
                 if pages[logical] != RELEASED:
                     group.pool.release(pages[logical])
                     pages[logical] = RELEASED

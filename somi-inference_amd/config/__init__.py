@@ -7,6 +7,8 @@ from .gizilorn import GizilornAttention, GizilornConfig, GizilornDense, Gizilorn
 from .kamedra import KamedraAttention, KamedraConfig, KamedraGLA, KamedraLayer, RotaryScaling
 from .metitar import (MetitarConfig, MetitarDense, MetitarExperts, MetitarHGRN2, MetitarLatentAttention, MetitarLayer,
                       RampedScaling)
+from .pusazen import (PusazenAttention, PusazenConfig, PusazenDense, PusazenExperts, PusazenLayer, PusazenLightning,
+                      PusazenMLSTM)
 from .qwen2 import Qwen2Config
 from .rusolorn import RusolornAttention, RusolornConfig, RusolornDeltaRule, RusolornExperts, RusolornLayer
 from .tomopel import (TomopelAttention, TomopelConfig, TomopelDense, TomopelExperts, TomopelLayer, TomopelMamba2,
@@ -19,7 +21,8 @@ __all__ = [
     "DEFAULT_NUM_BLOCKS", "EngineConfig", "GizilornAttention", "GizilornConfig", "GizilornDense",
     "GizilornLatentAttention", "GizilornLayer", "KamedraAttention", "KamedraConfig", "KamedraGLA", "KamedraLayer", "KeyReader",
     "MetitarConfig", "MetitarDense", "MetitarExperts", "MetitarHGRN2", "MetitarLatentAttention", "MetitarLayer", "RampedScaling",
-    "ModelConfig", "Qwen2Config", "RotaryScaling", "RusolornAttention", "RusolornConfig", "RusolornDeltaRule",
+    "ModelConfig", "PusazenAttention", "PusazenConfig", "PusazenDense", "PusazenExperts", "PusazenLayer", "PusazenLightning",
+    "PusazenMLSTM", "Qwen2Config", "RotaryScaling", "RusolornAttention", "RusolornConfig", "RusolornDeltaRule",
     "RusolornExperts", "RusolornLayer", "TomopelAttention", "TomopelConfig", "TomopelDense", "TomopelExperts", "TomopelLayer",
     "TomopelMamba2", "TomopelMinGRU", "TomopelParallel",
     "architecture_of", "config_from_dict", "normalize_dtype", "read_config_json",

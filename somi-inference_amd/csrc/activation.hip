@@ -275,3 +275,22 @@ extern "C" int somi_sigmoid_gate(const void* x, int dtype, const float* g, int64
     SOMI_LAUNCH_CHECK("sigmoid_gate");
     return 0;
 }
+
+// SiLU in place on the first `width` columns of rows row_stride apart (float32).
+__global__ void __launch_bounds__(256)
+silu_columns_kernel(float* __restrict__ rows, int64_t row_stride, int width) {
+    float* row = rows + (int64_t)blockIdx.x * row_stride;
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < width; c += gridDim.y * 256) {
+        const float v = row[c];
+        row[c] = v / (1.0f + expf(-v));
+    }
+}
+
+extern "C" int somi_silu_columns(float* rows, int64_t row_stride, int n_rows, int width, hipStream_t stream) {
+    SOMI_REQUIRE(n_rows >= 0 && width > 0 && row_stride >= width, "silu_columns: bad sizes");
+    if (n_rows == 0) return 0;
+    const int blocks = ceil_div(width, 1024);
+    hipLaunchKernelGGL(silu_columns_kernel, dim3(n_rows, blocks < 64 ? blocks : 64), dim3(256), 0, stream, rows, row_stride, width);
+    SOMI_LAUNCH_CHECK("silu_columns");
+    return 0;
+}

@@ -16,6 +16,7 @@
 // The wavefronts of a workgroup are merged through LDS; with several splits the workgroup writes
 // (max, sum, unnormalised output) to a workspace and a second kernel merges the splits in split order.
 #include "attention_bias.h"
+#include "attention_score.h"
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -251,17 +252,19 @@ __device__ __forceinline__ float lanes4_sum(float v) {
 // captured step of requests at 4,096 to 8,192 tokens allows) is one split, with four workgroups of head size 128 still
 // fitting a compute unit's LDS (38 KB each).
 #define DECODE_LDS_PAGES 768
-// BIAS: a distance bias is added to the scores (attention_bias.h); the rows of the workgroup's heads are in LDS where
-// they fit, in the units of the unscaled scores.
-template <int DT, bool BIAS>
+// FORM: SCORE_BIAS, a distance bias is added to the scores (attention_bias.h), and the rows of the workgroup's heads are in
+// LDS where they fit, in the units of the unscaled scores; SCORE_SHAPED, scores may be capped and cut into chunks and meet a
+// sink (attention_score.h).
+template <int DT, int FORM>
 __global__ void __launch_bounds__(256)
 attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc,
                             const bf16* __restrict__ vc, const int* __restrict__ block_table, int max_blocks,
                             const int* __restrict__ token_list, const int* __restrict__ token_entry,
                             const int* __restrict__ positions, int nq, int nkv, int page_size, int window,
-                            float scale, int split_len, int num_splits, DistanceBias bias, bf16* __restrict__ out,
-                            float* __restrict__ part_acc, float* __restrict__ part_ml) {
+                            float scale, int split_len, int num_splits, DistanceBias bias, ScoreShape shape,
+                            bf16* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml) {
     constexpr int D = DT * 16;
+    constexpr bool BIAS = FORM == SCORE_BIAS, SHAPED = FORM == SCORE_SHAPED;
     constexpr int QK_STEPS = (DT + 1) / 2;
     constexpr int KROW = D + 8, VROW = 32 + 4;               // padded LDS rows, in elements
     constexpr int K_CHUNKS = 32 * D / 8;                     // 16-byte pieces of a 32-key tile
@@ -284,14 +287,15 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
 
     const int p = positions[t];
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = SHAPED ? score_first_key(p, window, shape.chunk) : (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
     const int* table = block_table + (int64_t)token_entry[t] * max_blocks;
     int begin, end;                                  // this split's keys, inclusive
     decode_split_range(p, lo, split, split_len, num_splits, begin, end);
     const int hloc = hb * 16 + r;
     const int head = kvh * G + (hloc < G ? hloc : G - 1);
 
-    const float scale_log2 = scale * 1.44269504088896341f;
+    const ScoreCap cap(SHAPED ? shape.softcap : 0.f, scale * SCORE_LOG2E);
+    const float scale_log2 = SHAPED ? 1.0f : scale * 1.44269504088896341f;      // SHAPED: the scores are brought to base 2 at once
     float m_run = -INFINITY, l_run = 0.f;            // running maximum (in base-2 units) and sum
     f32x4 acc[MY_TILES];
 #pragma unroll
@@ -403,6 +407,12 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
                                                   : bias.table[(int64_t)head * bias.length + n] * inv_scale;
                     }
             }
+            if (SHAPED) {
+#pragma unroll
+                for (int half = 0; half < 2; ++half)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[half][i] = cap(s[half][i]);
+            }
             // s[half][i] = S[key j0 + 16 half + 4 g + i][head r], still unscaled; keys outside the split are
             // masked (only the first and last step of a split can hold any)
             if (j0 < begin || j0 + 31 > end) {
@@ -473,6 +483,8 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
     // acc[i][j] = O^T[d = (wave + 4 i) * 16 + 4 g + j][head r]; every wavefront holds the same m_run, l_run
     const int hq = kvh * G + hloc;
     if (hloc < G) {
+        if (SHAPED && num_splits == 1 && shape.sink != nullptr)
+            l_run += __builtin_amdgcn_exp2f(fmaf(shape.sink[hq], SCORE_LOG2E, -m_run));
 #pragma unroll
         for (int i = 0; i < MY_TILES; ++i) {
             const int dt = wave + 4 * i;
@@ -503,7 +515,7 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
 __global__ void __launch_bounds__(128)
 attention_combine_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                          const int* __restrict__ token_list, int nq, int D, int num_splits,
-                         bf16* __restrict__ out) {
+                         const float* __restrict__ sink, bf16* __restrict__ out) {
     __shared__ float factor[COMBINE_MAX_SPLITS];
     __shared__ float red[16];
     const int ti = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
@@ -520,7 +532,8 @@ attention_combine_kernel(const float* __restrict__ part_acc, const float* __rest
         factor[s] = f;
         lsum += l * f;
     }
-    const float l_all = block_sum<128>(lsum, red);      // also makes factor[] visible
+    float l_all = block_sum<128>(lsum, red);            // also makes factor[] visible
+    if (sink != nullptr) l_all += expf(sink[h] - m_all);
     // every split wrote its partial output (zeros where it saw no key), so the loads need no condition and
     // are issued eight at a time
     for (int d = tid; d < D; d += 128) {
@@ -550,7 +563,7 @@ template <int DT>
 static int launch_decode(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                          int max_blocks, const int* token_list, const int* token_entry, const int* positions,
                          int n_list, int nq, int nkv, int page_size, int window, float scale, int split_len,
-                         int num_splits, DistanceBias bias, void* out, float* part_acc, float* part_ml,
+                         int num_splits, DistanceBias bias, ScoreShape shape, void* out, float* part_acc, float* part_ml,
                          hipStream_t stream) {
     const int waves = DT <= 8 ? 4 : 2;
     const int G = nq / nkv, HB = (G + 15) / 16;
@@ -558,21 +571,29 @@ static int launch_decode(const void* q, int64_t q_stride, const void* kc, const 
     const bool pow2_pages = (page_size & (page_size - 1)) == 0;
     const bool staged = DT >= 2 && DT <= 8 && pow2_pages && n_list <= 65535 &&
                         split_len / page_size + 2 + 8 <= DECODE_LDS_PAGES;                        // + a tile's overhang
+    SOMI_REQUIRE(staged || !shape.any(), "attention_decode: capped, chunked and sinking scores come with head sizes 32 to 128, pages of a "
+                 "power of two keys and splits whose pages fit LDS (head size %d, pages of %d, splits of %d)", DT * 16, page_size, split_len);
     if (bias.length > 0) {
+        SOMI_REQUIRE(!shape.any(), "attention_decode: a distance bias does not come with capped, chunked or sinking scores");
         SOMI_REQUIRE(staged, "attention_decode: a distance bias comes with head sizes 32 to 128, pages of a power of two "
                      "keys and splits whose pages fit LDS (head size %d, pages of %d, splits of %d)", DT * 16, page_size, split_len);
         const int floats = (G < 16 ? G : 16) * bias.length;
         bias.in_lds = floats <= BIAS_LDS_FLOATS;
-        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), true>), dim3(nkv * HB, n_list, num_splits),
+        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), SCORE_BIAS>), dim3(nkv * HB, n_list, num_splits),
                            dim3(256), bias.in_lds ? floats * sizeof(float) : 0, stream, (const bf16*)q, q_stride,
                            (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, token_list, token_entry, positions,
-                           nq, nkv, page_size, window, scale, split_len, num_splits, bias, (bf16*)out, part_acc, part_ml);
-    } else if (staged)
-        // head sizes 32..128: keys and values staged through LDS (two tiles fit)
-        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), false>), dim3(nkv * HB, n_list, num_splits),
+                           nq, nkv, page_size, window, scale, split_len, num_splits, bias, shape, (bf16*)out, part_acc, part_ml);
+    } else if (shape.any()) {
+        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), SCORE_SHAPED>), dim3(nkv * HB, n_list, num_splits),
                            dim3(256), 0, stream, (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table,
                            max_blocks, token_list, token_entry, positions, nq, nkv, page_size, window, scale, split_len,
-                           num_splits, bias, (bf16*)out, part_acc, part_ml);
+                           num_splits, bias, shape, (bf16*)out, part_acc, part_ml);
+    } else if (staged)
+        // head sizes 32..128: keys and values staged through LDS (two tiles fit)
+        hipLaunchKernelGGL((attention_decode_lds_kernel<(DT >= 2 && DT <= 8 ? DT : 2), SCORE_PLAIN>), dim3(nkv * HB, n_list, num_splits),
+                           dim3(256), 0, stream, (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table,
+                           max_blocks, token_list, token_entry, positions, nq, nkv, page_size, window, scale, split_len,
+                           num_splits, bias, shape, (bf16*)out, part_acc, part_ml);
     else
         hipLaunchKernelGGL((attention_decode_kernel<DT>), dim3(n_list, nkv * HB, num_splits), dim3(waves * 64), smem,
                            stream, (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks,
@@ -581,7 +602,7 @@ static int launch_decode(const void* q, int64_t q_stride, const void* kc, const 
     SOMI_LAUNCH_CHECK("attention_decode");
     if (num_splits > 1) {
         hipLaunchKernelGGL(attention_combine_kernel, dim3(n_list, nq), dim3(128), 0, stream, part_acc, part_ml,
-                           token_list, nq, DT * 16, num_splits, (bf16*)out);
+                           token_list, nq, DT * 16, num_splits, shape.sink, (bf16*)out);
         SOMI_LAUNCH_CHECK("attention_combine");
     }
     return 0;
@@ -592,13 +613,14 @@ static int launch_decode(const void* q, int64_t q_stride, const void* kc, const 
 // page_size a multiple of 4.  k_cache [pages, nkv, page_size, D], v_cache [pages, nkv, D, page_size].
 // With num_splits > 1, part_acc holds n_list * nq * num_splits * D floats and part_ml
 // n_list * nq * num_splits * 2 floats; split_len is a multiple of 16 and split_len * num_splits covers every
-// listed token's position.  bias_table: [nq, bias_length] float32 or null (attention_bias.h).
+// listed token's position.  bias_table: [nq, bias_length] float32 or null (attention_bias.h); softcap, chunk, sink:
+// attention_score.h.
 extern "C" int somi_attention_decode(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                                      const int* block_table, int max_blocks, const int* token_list,
                                      const int* token_entry, const int* positions, int n_list, int nq, int nkv, int D,
                                      int page_size, int window, float scale, int split_len, int num_splits,
-                                     const float* bias_table, int bias_length, void* out, float* part_acc,
-                                     float* part_ml, hipStream_t stream) {
+                                     const float* bias_table, int bias_length, float softcap, int chunk, const float* sink,
+                                     void* out, float* part_acc, float* part_ml, hipStream_t stream) {
     SOMI_REQUIRE(n_list >= 0 && nq > 0 && nkv > 0 && max_blocks > 0, "attention_decode: bad sizes");
     SOMI_REQUIRE(nq % nkv == 0, "attention_decode: num_q_heads (%d) must be divisible by num_kv_heads (%d)", nq, nkv);
     SOMI_REQUIRE(D % 16 == 0 && D >= 16 && D <= 256, "attention_decode: head_dim %d must be a multiple of 16 up to 256", D);
@@ -614,11 +636,13 @@ extern "C" int somi_attention_decode(const void* q, int64_t q_stride, const void
     SOMI_REQUIRE(bias_length >= 0 && (bias_length == 0 || (bias_table != nullptr && scale > 0.f)),
                  "attention_decode: a distance bias needs its table and a scale above 0");
     if (n_list == 0) return 0;
+    SOMI_REQUIRE(softcap >= 0.f && chunk >= 0, "attention_decode: a soft cap of %g, chunks of %d", (double)softcap, chunk);
     const DistanceBias bias{bias_table, bias_length, 0};
+    const ScoreShape shape{softcap, chunk, sink};
 #define SOMI_DECODE(DT)                                                                                              \
     case DT:                                                                                                         \
         return launch_decode<DT>(q, q_stride, k_cache, v_cache, block_table, max_blocks, token_list, token_entry,    \
-                                 positions, n_list, nq, nkv, page_size, window, scale, split_len, num_splits, bias, out, \
+                                 positions, n_list, nq, nkv, page_size, window, scale, split_len, num_splits, bias, shape, out, \
                                  part_acc, part_ml, stream)
     switch (D / 16) {
         SOMI_DECODE(1); SOMI_DECODE(2); SOMI_DECODE(3); SOMI_DECODE(4); SOMI_DECODE(5); SOMI_DECODE(6);

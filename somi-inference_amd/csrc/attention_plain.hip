@@ -11,8 +11,10 @@
 // aligned to absolute positions, so the arithmetic for a (request, position) is the same
 // whatever portion or batch the token arrives in.  Everything is float32.
 //
-// A distance bias (attention_bias.h) may be added to the scaled scores.
+// A distance bias (attention_bias.h) may be added to the scaled scores; they may be capped, cut into chunks and meet a
+// sink (attention_score.h).
 #include "attention_bias.h"
+#include "attention_score.h"
 #include "common.h"
 
 template <typename T, int NT>
@@ -21,7 +23,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int64_t q_stride, const T*
                              const T* __restrict__ vc, const int* __restrict__ block_table, int max_blocks,
                              const int* __restrict__ token_entry, const int* __restrict__ positions, int nq,
                              int nkv, int D, int page_size, int window, float scale, DistanceBias bias,
-                             T* __restrict__ out) {
+                             ScoreShape shape, T* __restrict__ out) {
     extern __shared__ float smem[];
     float* qs = smem;                          // [D]
     float* ps = qs + ((D + 1) & ~1);           // [NT] softmax weights of the tile
@@ -33,7 +35,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int64_t q_stride, const T*
     const int e = token_entry[t];
     const int p = positions[t];
     const int kvh = h / (nq / nkv);
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = score_first_key(p, window, shape.chunk);
     const int* table = block_table + (int64_t)e * max_blocks;
 
     for (int d = tid; d < D; d += NT) qs[d] = to_float(q[(int64_t)t * q_stride + (int64_t)h * D + d]);
@@ -55,6 +57,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int64_t q_stride, const T*
             float dot = 0.f;
             for (int d = 0; d < D; ++d) dot = fmaf(qs[d], to_float(kr[d]), dot);
             s = dot * scale;
+            if (shape.softcap > 0.f) s = shape.softcap * tanhf(s / shape.softcap);
             if (p - pos < bias.length) s += bias.table[(int64_t)h * bias.length + (p - pos)];
         }
         const float tile_max = block_max<NT>(s, red);
@@ -78,6 +81,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int64_t q_stride, const T*
             }
         }
     }
+    if (shape.sink != nullptr) l += expf(shape.sink[h] - m);
 #pragma unroll
     for (int r = 0; r < 2; ++r) {
         const int d = tid + r * NT;
@@ -89,12 +93,13 @@ paged_attention_plain_kernel(const T* __restrict__ q, int64_t q_stride, const T*
 // v_cache: [num_pages, nkv, D, page_size].
 // block_table: [n_entries, max_blocks] int32 page ids of each entry's request (pages a window has passed
 // may hold -1; they are never read).  token_entry, positions: [n_tokens] int32.  bias: [nq, bias_length] float32 or
-// null (attention_bias.h).  out: [n_tokens, nq * D].
+// null (attention_bias.h).  softcap, chunk, sink: attention_score.h.  out: [n_tokens, nq * D].
 extern "C" int somi_paged_attention_plain(const void* q, int dtype, int64_t q_stride, const void* k_cache,
                                           const void* v_cache, const int* block_table, int max_blocks,
                                           const int* token_entry, const int* positions, int n_tokens, int nq,
                                           int nkv, int D, int page_size, int window, float scale,
-                                          const float* bias, int bias_length, void* out, hipStream_t stream) {
+                                          const float* bias, int bias_length, float softcap, int chunk,
+                                          const float* sink, void* out, hipStream_t stream) {
     constexpr int NT = 128;
     SOMI_REQUIRE(n_tokens >= 0 && nq > 0 && nkv > 0 && D > 0 && page_size > 0 && max_blocks > 0,
                  "paged_attention: bad sizes");
@@ -102,7 +107,9 @@ extern "C" int somi_paged_attention_plain(const void* q, int dtype, int64_t q_st
     SOMI_REQUIRE(D <= 2 * NT, "paged_attention: head_dim %d is larger than the supported %d", D, 2 * NT);
     SOMI_REQUIRE(window >= 0, "paged_attention: window must be >= 0");
     SOMI_REQUIRE(bias_length >= 0 && (bias_length == 0 || bias != nullptr), "paged_attention: a distance bias needs its table");
+    SOMI_REQUIRE(softcap >= 0.f && chunk >= 0, "paged_attention: a soft cap of %g, chunks of %d", (double)softcap, chunk);
     const DistanceBias table{bias, bias_length};
+    const ScoreShape shape{softcap, chunk, sink};
     SOMI_REQUIRE(nq <= 65535, "paged_attention: too many heads");
     if (n_tokens == 0) return 0;
     const dim3 grid(n_tokens, nq);
@@ -110,11 +117,11 @@ extern "C" int somi_paged_attention_plain(const void* q, int dtype, int64_t q_st
     if (dtype == SOMI_F32)
         hipLaunchKernelGGL((paged_attention_plain_kernel<float, NT>), grid, dim3(NT), smem, stream, (const float*)q,
                            q_stride, (const float*)k_cache, (const float*)v_cache, block_table, max_blocks,
-                           token_entry, positions, nq, nkv, D, page_size, window, scale, table, (float*)out);
+                           token_entry, positions, nq, nkv, D, page_size, window, scale, table, shape, (float*)out);
     else if (dtype == SOMI_BF16)
         hipLaunchKernelGGL((paged_attention_plain_kernel<bf16, NT>), grid, dim3(NT), smem, stream, (const bf16*)q,
                            q_stride, (const bf16*)k_cache, (const bf16*)v_cache, block_table, max_blocks,
-                           token_entry, positions, nq, nkv, D, page_size, window, scale, table, (bf16*)out);
+                           token_entry, positions, nq, nkv, D, page_size, window, scale, table, shape, (bf16*)out);
     else
         return somi_fail("paged_attention: unknown dtype %d", dtype);
     SOMI_LAUNCH_CHECK("paged_attention_plain");

@@ -18,6 +18,7 @@
 // Every key tile is used for all QB query blocks from registers.  Key tiles are aligned to absolute
 // positions (multiples of 32), so a query's arithmetic does not depend on how the prompt was cut.
 #include "attention_bias.h"
+#include "attention_score.h"
 #include "common.h"
 #include "attention_prefill_tile.h"
 
@@ -254,15 +255,20 @@ static int prefill_key_split_below(int units) { return 7 * units / 2; }      // 
 // KS = 2: twice the wavefronts; each query block is owned by KS of them, which take the 32-key tiles in turn
 // (tile index modulo KS, by absolute position) and join their sums, maxima and outputs through LDS at the
 // end.  The longest workgroup, which sets the time of a short prompt, has half as many steps to walk.
-// BIAS: a distance bias is added to the scores (attention_bias.h); its head's row is in LDS behind the page list where it
-// fits, in the units of the unscaled scores.
-template <int DT, int QB, int KS, bool BIAS>
+// FORM: SCORE_BIAS, a distance bias is added to the scores (attention_bias.h), its head's row in LDS behind the page list
+// where it fits, in the units of the unscaled scores; SCORE_SHAPED, scores may be capped and cut into chunks and meet a sink
+// (attention_score.h).
+template <int DT, int QB, int KS, int FORM>
 __global__ void __launch_bounds__(256 * KS, 2 * KS)     // the second figure: wavefronts per SIMD to leave room for
 attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc,
                              const bf16* __restrict__ vc, const int* __restrict__ block_table, int max_blocks,
                              const int* __restrict__ entry_start, const int* __restrict__ entry_first_pos, const int* __restrict__ entry_len, int nq,
-                             int nkv, int page_size, int window, float scale_log2, DistanceBias bias, int bias_at, bf16* __restrict__ out) {
+                             int nkv, int page_size, int window, float scale_log2_, DistanceBias bias, int bias_at, ScoreShape shape,
+                             bf16* __restrict__ out) {
     constexpr int D = DT * 16;
+    constexpr bool BIAS = FORM == SCORE_BIAS, SHAPED = FORM == SCORE_SHAPED;
+    const ScoreCap cap(SHAPED ? shape.softcap : 0.f, scale_log2_);
+    const float scale_log2 = SHAPED ? 1.0f : scale_log2_;               // SHAPED: the scores are brought to base 2 at once
     constexpr int QK_STEPS = (DT + 1) / 2;
     constexpr int QW = QB * 16, WAVES = 4, QG = WAVES * QW;             // 64 or 128 queries per workgroup
     constexpr int KROW = D + 8, VROW = 32 + 4;                          // padded LDS rows, in elements
@@ -295,7 +301,7 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
     const int* table = block_table + (int64_t)e * max_blocks;
     const int wg_valid = len - g0 < QG ? len - g0 : QG;
     const int wg_first = pos0 + g0, wg_last = pos0 + g0 + wg_valid - 1;
-    const int lo = (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
+    const int lo = SHAPED ? score_first_key(wg_first, window, shape.chunk) : (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
     const int vlo = lo & ~3, vhi = wg_last & ~3;
 
     // The pages of the visible range go to LDS once, so that a tile's addresses do not wait for a
@@ -327,13 +333,17 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
     const bool active = q0 < len;
     const int nvalid = active ? (len - q0 < QW ? len - q0 : QW) : 0;
     const int w_last = pos0 + q0 + nvalid - 1;
+    // SHAPED: the first key that each query sees, that the wavefront's first query sees, and that its last one sees
+    const int w_lo = SHAPED && active ? score_first_key(pos0 + q0, window, shape.chunk) : 0;
+    const int w_edge = SHAPED && active ? score_first_key(w_last, window, shape.chunk) : 0;
     bf16x8 qf[QB][QK_STEPS];
-    int pcol[QB];
+    int pcol[QB], first_key[QB];
 #pragma unroll
     for (int qb = 0; qb < QB; ++qb) {
         int qi = q0 + qb * 16 + r;
         qi = qi < len ? qi : len - 1;
         pcol[qb] = pos0 + qi;
+        first_key[qb] = SHAPED ? score_first_key(pcol[qb], window, shape.chunk) : 0;
         const bf16* qrow = q + (int64_t)(start + qi) * q_stride + (int64_t)h * D;
 #pragma unroll
         for (int c = 0; c < DT / 2; ++c) qf[qb][c] = pld8(qrow + c * 32 + g * 8);
@@ -411,7 +421,7 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
         const bool more = j_step + STEP <= wg_last;
         if (j_step + 2 * STEP <= wg_last) fetch(kfree, vfree, j_step + 2 * STEP);
         const int j0 = j_step + 32 * kh;                     // this wavefront's tile of the step
-        if (active && j0 <= w_last) {
+        if (active && j0 <= w_last && (!SHAPED || j0 + 31 >= w_lo)) {
             bf16x8 kf[2][QK_STEPS];
 #pragma unroll
             for (int half = 0; half < 2; ++half) {
@@ -447,13 +457,21 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
                             s[qb][half][i] += bias.in_lds ? bias_s[n] : bias_row[n] * bias_unit;
                         }
             }
+            if (SHAPED) {
+#pragma unroll
+                for (int qb = 0; qb < QB; ++qb)
+#pragma unroll
+                    for (int half = 0; half < 2; ++half)
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) s[qb][half][i] = cap(s[qb][half][i]);
+            }
             // scores stay unscaled; keys a query must not see are masked, which only steps that reach past the
-            // wavefront's first query (or a window's lower edge) can hold
-            if (window > 0 || j0 + 31 > pos0 + q0) {
+            // wavefront's first query (or a window's or a chunk's lower edge) can hold
+            if ((SHAPED ? j0 < w_edge : window > 0) || j0 + 31 > pos0 + q0) {
 #pragma unroll
                 for (int qb = 0; qb < QB; ++qb) {
                     const int p = pcol[qb];
-                    const int first = window > 0 ? p - window + 1 : 0;
+                    const int first = SHAPED ? first_key[qb] : window > 0 ? p - window + 1 : 0;
 #pragma unroll
                     for (int half = 0; half < 2; ++half)
 #pragma unroll
@@ -551,6 +569,7 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
             const float m_use = m_new == -INFINITY ? 0.f : m_new;
             const float mine = __builtin_amdgcn_exp2f(m_run[qb] - m_use), theirs = __builtin_amdgcn_exp2f(m_other - m_use);
             l_run[qb] = l_run[qb] * mine + l_other * theirs;
+            m_run[qb] = m_use;
 #pragma unroll
             for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
@@ -558,10 +577,12 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
         }
     }
     if (!active) return;
+    const float sink = SHAPED && shape.sink != nullptr ? shape.sink[h] * SCORE_LOG2E : -INFINITY;
 #pragma unroll
     for (int qb = 0; qb < QB; ++qb) {
         const int qi = q0 + qb * 16 + r;
         if (qi >= len) continue;
+        if (SHAPED) l_run[qb] += __builtin_amdgcn_exp2f(sink - m_run[qb]);
         const float inv = 1.0f / l_run[qb];
         bf16* orow = out + ((int64_t)(start + qi) * nq + h) * D + g * 4;
 #pragma unroll
@@ -577,6 +598,9 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
 // before its last query, or a window and the workgroup's 128 queries) and a 32-key tile's overhang.
 // Static LDS of the LDS kernel: two buffers of KS key tiles [32][D + 8] and value tiles [D][36], bfloat16.
 static int prefill_lds_static(int D, int ks) { return 2 * ks * (32 * (D + 8) + D * 36) * 2; }
+
+// How many keys before a workgroup's first query it may have to walk: a window's or a chunk's, 0 for all.
+static int score_reach(int window, int chunk) { return window > 0 && chunk > 0 ? min(window, chunk) : max(window, chunk); }
 
 static int prefill_page_entries(int max_blocks, int page_size, int window) {
     int entries = max_blocks + 16;                   // + the overhang of a step of two 32-key tiles, pages of 4 keys
@@ -607,35 +631,43 @@ template <int DT>
 static int launch_prefill_lds(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                               int max_blocks, const int* entry_start, const int* entry_first_pos, const int* entry_len, int n_entries,
                               int max_entry_len, int max_context, int shape, int nq, int nkv, int page_size,
-                              int window, float scale, DistanceBias bias, void* out, hipStream_t stream) {
-    const int bias_at = prefill_page_entries(max_blocks, page_size, window);
+                              int window, float scale, DistanceBias bias, ScoreShape score, void* out, hipStream_t stream) {
+    const int reach = score_reach(window, score.chunk);
+    const int bias_at = prefill_page_entries(max_blocks, page_size, reach);
     size_t page_list = (size_t)bias_at * sizeof(int);             // dynamic LDS: the page list, then the bias if it fits
     bias.in_lds = bias.length > 0 && bias.length <= BIAS_LDS_FLOATS &&
                   (int)page_list + bias.length * 4 + prefill_lds_static(DT * 16, 1) <= PREFILL_LDS_TOTAL;
     if (bias.in_lds) page_list += bias.length * sizeof(float);
     const bool split_fits = (int)page_list + prefill_lds_static(DT * 16, 2) <= PREFILL_LDS_TOTAL;
     if (shape == PREFILL_SHAPE_AUTO)
-        shape = prefill_lds_choice(n_entries, max_entry_len, max_context, nq, window, split_fits, somi_units());
+        shape = prefill_lds_choice(n_entries, max_entry_len, max_context, nq, reach, split_fits, somi_units());
     const bool wide = shape == PREFILL_SHAPE_WIDE;
     const dim3 grid(nq, n_entries, ceil_div(max_entry_len, wide ? 128 : 64));
-#define PREFILL_LDS_LAUNCH(QB, KS, BIAS)                                                                                    \
+#define PREFILL_LDS_LAUNCH(QB, KS, FORM)                                                                                    \
     do {                                                                                                                    \
         if (page_list > 16 * 1024)                       /* with the tiles beyond the default limit of LDS */               \
-            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, QB, KS, BIAS>,                          \
+            (void)hipFuncSetAttribute((const void*)attention_prefill_lds_kernel<DT, QB, KS, FORM>,                          \
                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)page_list);                          \
-        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, QB, KS, BIAS>), grid, dim3(256 * KS), page_list, stream,       \
+        hipLaunchKernelGGL((attention_prefill_lds_kernel<DT, QB, KS, FORM>), grid, dim3(256 * KS), page_list, stream,       \
                            (const bf16*)q, q_stride, (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start, \
                            entry_first_pos, entry_len, nq, nkv, page_size, window, scale * 1.44269504088896341f, bias,      \
-                           bias_at, (bf16*)out);                                                                            \
+                           bias_at, score, (bf16*)out);                                                                     \
+    } while (0)
+#define PREFILL_LDS_FORM(QB, KS)                                                                                            \
+    do {                                                                                                                    \
+        if (bias.length > 0) PREFILL_LDS_LAUNCH(QB, KS, SCORE_BIAS);                                                        \
+        else if (score.any()) PREFILL_LDS_LAUNCH(QB, KS, SCORE_SHAPED);                                                     \
+        else PREFILL_LDS_LAUNCH(QB, KS, SCORE_PLAIN);                                                                       \
     } while (0)
     if (wide) {
-        if (bias.length > 0) PREFILL_LDS_LAUNCH(2, 1, true); else PREFILL_LDS_LAUNCH(2, 1, false);
+        PREFILL_LDS_FORM(2, 1);
     } else if (shape == PREFILL_SHAPE_SPLIT && split_fits) {
         // few workgroups with many tiles each: the keys of a query block are split over two wavefronts
-        if (bias.length > 0) PREFILL_LDS_LAUNCH(1, 2, true); else PREFILL_LDS_LAUNCH(1, 2, false);
+        PREFILL_LDS_FORM(1, 2);
     } else {
-        if (bias.length > 0) PREFILL_LDS_LAUNCH(1, 1, true); else PREFILL_LDS_LAUNCH(1, 1, false);
+        PREFILL_LDS_FORM(1, 1);
     }
+#undef PREFILL_LDS_FORM
 #undef PREFILL_LDS_LAUNCH
     SOMI_LAUNCH_CHECK("attention_prefill_lds");
     return 0;
@@ -663,12 +695,14 @@ static int launch_prefill(const void* q, int64_t q_stride, const void* kc, const
 // up to 256; page_size a multiple of 4.  k_cache [pages, nkv, page_size, D], v_cache [pages, nkv, D, page_size];
 // out: [n_tokens, nq * D].  max_context: the longest context a portion ends at (a hint for the launch shape; 0: unknown).
 // shape: 0 lets the launcher choose; 1..3 ask for a launch shape of the 16 x 16 LDS kernel, 4 and 5 for one of the
-// 32 x 32 tile kernel (PREFILL_SHAPE_*).  bias_table: [nq, bias_length] float32 or null (attention_bias.h).
+// 32 x 32 tile kernel (PREFILL_SHAPE_*).  bias_table: [nq, bias_length] float32 or null (attention_bias.h);
+// softcap, chunk, sink: attention_score.h.
 extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const void* k_cache, const void* v_cache,
                                       const int* block_table, int max_blocks, const int* entry_start,
                                       const int* entry_first_pos, const int* entry_len, int n_entries, int max_entry_len, int max_context,
                                       int shape, int nq, int nkv, int D, int page_size, int window, float scale,
-                                      const float* bias_table, int bias_length, void* out, hipStream_t stream) {
+                                      const float* bias_table, int bias_length, float softcap, int chunk, const float* sink,
+                                      void* out, hipStream_t stream) {
     SOMI_REQUIRE(n_entries >= 0 && max_entry_len >= 0 && nq > 0 && nkv > 0 && max_blocks > 0,
                  "attention_prefill: bad sizes");
     SOMI_REQUIRE(nq % nkv == 0, "attention_prefill: num_q_heads (%d) must be divisible by num_kv_heads (%d)", nq, nkv);
@@ -685,9 +719,13 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
     SOMI_REQUIRE(bias_length >= 0 && (bias_length == 0 || (bias_table != nullptr && scale > 0.f)),
                  "attention_prefill: a distance bias needs its table and a scale above 0");
     if (n_entries == 0 || max_entry_len == 0) return 0;
+    SOMI_REQUIRE(softcap >= 0.f && chunk >= 0, "attention_prefill: a soft cap of %g, chunks of %d", (double)softcap, chunk);
     const DistanceBias bias{bias_table, bias_length, 0};
+    const ScoreShape score{softcap, chunk, sink};
+    SOMI_REQUIRE(bias_length == 0 || !score.any(), "attention_prefill: a distance bias does not come with capped, chunked or sinking scores");
+    const int reach = score_reach(window, chunk);
     // head sizes 64 and 128 over pages of 8 keys or more: the 32 x 32 tile kernel
-    const bool tile_ok = somi_prefill_tile_applies(D, page_size, max_blocks, window) && (uintptr_t)v_cache % 16 == 0;
+    const bool tile_ok = somi_prefill_tile_applies(D, page_size, max_blocks, reach) && (uintptr_t)v_cache % 16 == 0;
     if (shape >= PREFILL_SHAPE_TILE)
         SOMI_REQUIRE(tile_ok, "attention_prefill: the tile kernel does not take head size %d, pages of %d keys or a block table of %d pages",
                      D, page_size, max_blocks);
@@ -695,7 +733,7 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
         const int64_t groups = (int64_t)ceil_div(max_entry_len, 256) * n_entries * nq;
         const bool wide = shape == PREFILL_SHAPE_AUTO ? groups >= prefill_tile_wide_groups(somi_units()) : shape == PREFILL_SHAPE_TILE_WIDE;
         return somi_prefill_tile(q, q_stride, k_cache, v_cache, block_table, max_blocks, entry_start, entry_first_pos, entry_len,
-                                 n_entries, max_entry_len, wide, nq, nkv, D, page_size, window, scale, bias, out, stream);
+                                 n_entries, max_entry_len, wide, nq, nkv, D, page_size, window, scale, bias, score, out, stream);
     }
 #define SOMI_PREFILL(DT, QB)                                                                                       \
     case DT:                                                                                                       \
@@ -710,14 +748,14 @@ extern "C" int somi_attention_prefill(const void* q, int64_t q_stride, const voi
                                          scale, out, stream);                                                      \
         return launch_prefill_lds<DT>(q, q_stride, k_cache, v_cache, block_table, max_blocks, entry_start,         \
                                       entry_first_pos, entry_len, n_entries, max_entry_len, max_context, shape, nq, nkv,      \
-                                      page_size, window, scale, bias, out, stream)
+                                      page_size, window, scale, bias, score, out, stream)
     // head sizes 32..128 stage keys and values through LDS; the others (LDS would not hold two tiles, or a
     // tile is smaller than the workgroup's loads) keep them in registers per wavefront, and so do page sizes
     // that are no power of two and block tables too wide for the LDS copy of a request's pages
     const bool lds_ok = (page_size & (page_size - 1)) == 0 &&
-                        prefill_page_entries(max_blocks, page_size, window) * 4 + prefill_lds_static(D, 1) <= PREFILL_LDS_TOTAL;
-    SOMI_REQUIRE(bias_length == 0 || (lds_ok && D >= 32 && D <= 128),
-                 "attention_prefill: a distance bias comes with head sizes 32 to 128 and pages of a power of two keys whose "
+                        prefill_page_entries(max_blocks, page_size, reach) * 4 + prefill_lds_static(D, 1) <= PREFILL_LDS_TOTAL;
+    SOMI_REQUIRE((bias_length == 0 && !score.any()) || (lds_ok && D >= 32 && D <= 128),
+                 "attention_prefill: a distance bias and capped, chunked or sinking scores come with head sizes 32 to 128 and pages of a power of two keys whose "
                  "list fits LDS (head size %d, pages of %d)", D, page_size);
     switch (D / 16) {
         SOMI_PREFILL(1, 4); SOMI_PREFILL_LDS(2); SOMI_PREFILL_LDS(3); SOMI_PREFILL_LDS(4); SOMI_PREFILL_LDS(5);
@@ -743,7 +781,7 @@ extern "C" int somi_attention_prefill_choice(int n_entries, int max_entry_len, i
     return prefill_lds_choice(n_entries, max_entry_len, max_context, nq, window, split_fits != 0, units);
 }
 
-// Whether the matrix-core kernels take a distance bias at these sizes: both the prompts' and the decoded tokens' kernel
+// Whether the matrix-core kernels take a distance bias, or capped, chunked and sinking scores, at these sizes: both the prompts' and the decoded tokens' kernel
 // must be one of those that stage keys through LDS.
 extern "C" int somi_attention_bias_supported(int D, int page_size, int max_blocks) {
     if (D % 16 != 0 || D < 32 || D > 128 || page_size < 4 || (page_size & (page_size - 1)) != 0) return 0;

@@ -4,6 +4,7 @@
 #include <hip/hip_runtime.h>
 #include <stdint.h>
 #include "attention_bias.h"
+#include "attention_score.h"
 
 #define SOMI_PREFILL_TILE_LDS_MAX (112 * 1024)   // dynamic LDS a workgroup of the kernel may ask for (launches with 106 KB are tested)
 
@@ -16,4 +17,4 @@ bool somi_prefill_tile_applies(int D, int page_size, int max_blocks, int window)
 int somi_prefill_tile(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                       int max_blocks, const int* entry_start, const int* entry_first_pos, const int* entry_len,
                       int n_entries, int max_entry_len, bool wide, int nq, int nkv, int D, int page_size, int window,
-                      float scale, DistanceBias bias, void* out, hipStream_t stream);
+                      float scale, DistanceBias bias, ScoreShape score, void* out, hipStream_t stream);

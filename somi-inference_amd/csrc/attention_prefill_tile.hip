@@ -63,15 +63,19 @@ __device__ __forceinline__ float tile_pair_max(float v) {
 }
 
 // D: head size (64 or 128).  QBLK query blocks of 32 per workgroup, KS key splits; QBLK * KS wavefronts.
-// BIAS: a distance bias is added to the scores (attention_bias.h); its head's row is in LDS behind the page list where it
-// fits, in the units of the score product.
-template <int D, int QBLK, int KS, bool BIAS>
+// FORM: SCORE_BIAS, a distance bias is added to the scores (attention_bias.h), its head's row in LDS behind the page list
+// where it fits, in the units of the score product; SCORE_SHAPED, scores may be capped and cut into chunks and meet a sink
+// (attention_score.h): a capped score is no longer linear in the product, so the reference point is subtracted after it.
+template <int D, int QBLK, int KS, int FORM>
 __global__ void __launch_bounds__(QBLK * KS * 64, 2)
 prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ kc, const bf16* __restrict__ vc,
                     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ entry_start,
                     const int* __restrict__ entry_first_pos, const int* __restrict__ entry_len, int nq, int nkv,
-                    int page_size, int window, float scale_pow2, float scale_rest, DistanceBias bias, int bias_at,
-                    bf16* __restrict__ out) {
+                    int page_size, int window, float scale_pow2, float scale_rest_, DistanceBias bias, int bias_at,
+                    ScoreShape shape, bf16* __restrict__ out) {
+    constexpr bool BIAS = FORM == SCORE_BIAS, SHAPED = FORM == SCORE_SHAPED;
+    const ScoreCap cap(SHAPED ? shape.softcap : 0.f, scale_rest_);
+    const float scale_rest = SHAPED ? 1.0f : scale_rest_;        // SHAPED: the scores are brought to base 2 at once
     constexpr int THREADS = QBLK * KS * 64;
     constexpr int CH = D / 8;                    // 16-byte pieces of a key row
     constexpr int KROW = D * 2;                  // bytes
@@ -99,7 +103,7 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
     const int* table = block_table + (int64_t)e * max_blocks;
     const int wg_valid = len - g0 < QG ? len - g0 : QG;
     const int wg_first = pos0 + g0, wg_last = pos0 + g0 + wg_valid - 1;
-    const int lo = (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
+    const int lo = SHAPED ? score_first_key(wg_first, window, shape.chunk) : (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
 
     const int shift = __builtin_ctz(page_size);
     const int j_begin = lo & ~(STEP - 1);
@@ -177,11 +181,12 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
     const bool active = q0 < len;
     const int nvalid = active ? (len - q0 < 32 ? len - q0 : 32) : 0;
     const int w_first = pos0 + q0, w_last = pos0 + q0 + nvalid - 1;
-    const int w_lo = (window > 0 && w_first - window + 1 > 0) ? w_first - window + 1 : 0;
+    const int w_lo = SHAPED ? score_first_key(w_first, window, shape.chunk) : (window > 0 && w_first - window + 1 > 0) ? w_first - window + 1 : 0;
+    const int w_edge = SHAPED ? score_first_key(w_last > 0 ? w_last : 0, window, shape.chunk) : 0;     // what the last query sees first
     int qi = q0 + col;
     qi = qi < len ? qi : len - 1;
     const int p = pos0 + qi;                              // this lane's query position
-    const int p_first = window > 0 ? p - window + 1 : 0;
+    const int p_first = SHAPED ? score_first_key(p, window, shape.chunk) : window > 0 ? p - window + 1 : 0;
     bf16x8 qf[KSTEPS];
     {
         const bf16* qrow = q + (int64_t)(start + qi) * q_stride + (int64_t)h * D;
@@ -261,13 +266,18 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
                     for (int r = 0; r < 16; ++r) sc[r] += bias_row[bias_index(n0 - (16 * (r >> 3) + (r & 7)), bias.length)] * bias_unit;
                 }
             }
+            if (SHAPED) {
+                const float point = m_run == -INFINITY ? 0.f : m_run;
+#pragma unroll
+                for (int r = 0; r < 16; ++r) sc[r] = cap(sc[r]) - point;
+            }
             if (j0 + 31 > w_first) {
                 const int lim = p_rel - j0;
 #pragma unroll
                 for (int r = 0; r < 16; ++r)
                     if (16 * (r >> 3) + (r & 7) > lim) sc[r] = -INFINITY;
             }
-            if (window > 0) {
+            if (SHAPED ? j0 < w_edge : window > 0) {
                 const int first = p_first - j0 - 8 * hf;
 #pragma unroll
                 for (int r = 0; r < 16; ++r)
@@ -290,7 +300,7 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
 #pragma unroll
                     for (int r = 0; r < 16; ++r) acc[b][r] *= corr;
                 acc_l[0] *= corr;
-                const float neg = m_run == -INFINITY ? 0.f : -m_run;
+                const float neg = SHAPED || m_run == -INFINITY ? 0.f : -m_run;
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     sc[r] -= delta;
@@ -366,12 +376,14 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
         const float mine = __builtin_amdgcn_exp2f((m_run - m_use) * scale_rest);
         const float theirs = __builtin_amdgcn_exp2f((m_other - m_use) * scale_rest);
         l_run = l_run * mine + l_other * theirs;
+        m_run = m_use;
 #pragma unroll
         for (int b = 0; b < DBLK; ++b)
 #pragma unroll
             for (int r = 0; r < 16; ++r) acc[b][r] = acc[b][r] * mine + hand[(b * 16 + r) * 64] * theirs;
     }
     if (!active || q0 + col >= len) return;
+    if (SHAPED && shape.sink != nullptr) l_run += __builtin_amdgcn_exp2f(fmaf(shape.sink[h], SCORE_LOG2E, -m_run));
     // register r of block b: channel 32 b + 8 (r / 4) + 4 hf + r % 4
     const float inv = 1.0f / l_run;
     bf16* orow = out + ((int64_t)(start + q0 + col) * nq + h) * D + 4 * hf;
@@ -391,22 +403,24 @@ static int tile_page_entries(int qblk, int max_blocks, int page_size, int window
     return window > 0 ? min(entries, (window + qblk * 32 + 128) / page_size + 4) : entries;
 }
 
-template <int D, int QBLK, int KS, bool BIAS>
+template <int D, int QBLK, int KS, int FORM>
 static int launch_tile(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table, int max_blocks,
                        const int* entry_start, const int* entry_first_pos, const int* entry_len, int n_entries,
                        int max_entry_len, int nq, int nkv, int page_size, int window, float scale, DistanceBias bias,
-                       void* out, hipStream_t stream) {
+                       ScoreShape score, void* out, hipStream_t stream) {
+    constexpr bool BIAS = FORM == SCORE_BIAS;
+    const int reach = window > 0 && score.chunk > 0 ? min(window, score.chunk) : max(window, score.chunk);     // sizes the page list
     // dynamic LDS: the stages and the page list, then (BIAS) the head's row if it fits
-    const int bias_at = tile_page_entries(QBLK, max_blocks, page_size, window);
+    const int bias_at = tile_page_entries(QBLK, max_blocks, page_size, reach);
     const int with_bias = 2 * KS * (32 * D * 2 + D * 64) + (bias_at + bias.length) * 4;
-    int lds = somi_prefill_tile_lds(D, QBLK, KS, max_blocks, page_size, window);
+    int lds = somi_prefill_tile_lds(D, QBLK, KS, max_blocks, page_size, reach);
     bias.in_lds = BIAS && bias.length <= BIAS_LDS_FLOATS && with_bias <= SOMI_PREFILL_TILE_LDS_MAX;
     if (bias.in_lds) lds = max(lds, with_bias);
     static int lds_allowed[64];                  // per device: the largest dynamic LDS this kernel has been allowed so far
     int device = 0;
     if (hipGetDevice(&device) != hipSuccess || device < 0 || device >= 64) return somi_fail("attention_prefill_tile: hipGetDevice failed");
     if (lds > lds_allowed[device]) {
-        const hipError_t err = hipFuncSetAttribute((const void*)prefill_tile_kernel<D, QBLK, KS, BIAS>,
+        const hipError_t err = hipFuncSetAttribute((const void*)prefill_tile_kernel<D, QBLK, KS, FORM>,
                                                    hipFuncAttributeMaxDynamicSharedMemorySize, lds);
         if (err != hipSuccess) return somi_fail("attention_prefill_tile: %d bytes of LDS refused: %s", lds, hipGetErrorString(err));
         lds_allowed[device] = lds;
@@ -416,9 +430,9 @@ static int launch_tile(const void* q, int64_t q_stride, const void* kc, const vo
     int exponent = 0;
     const float rest = 2.f * frexpf(scale * 1.44269504088896341f, &exponent);
     const float pow2 = ldexpf(1.f, exponent - 1);
-    hipLaunchKernelGGL((prefill_tile_kernel<D, QBLK, KS, BIAS>), grid, dim3(QBLK * KS * 64), lds, stream, (const bf16*)q, q_stride,
+    hipLaunchKernelGGL((prefill_tile_kernel<D, QBLK, KS, FORM>), grid, dim3(QBLK * KS * 64), lds, stream, (const bf16*)q, q_stride,
                        (const bf16*)kc, (const bf16*)vc, block_table, max_blocks, entry_start, entry_first_pos, entry_len,
-                       nq, nkv, page_size, window, pow2, rest, bias, bias_at, (bf16*)out);
+                       nq, nkv, page_size, window, pow2, rest, bias, bias_at, score, (bf16*)out);
     SOMI_LAUNCH_CHECK("attention_prefill_tile");
     return 0;
 }
@@ -443,15 +457,16 @@ bool somi_prefill_tile_applies(int D, int page_size, int max_blocks, int window)
 int somi_prefill_tile(const void* q, int64_t q_stride, const void* kc, const void* vc, const int* block_table,
                       int max_blocks, const int* entry_start, const int* entry_first_pos, const int* entry_len,
                       int n_entries, int max_entry_len, bool wide, int nq, int nkv, int D, int page_size, int window,
-                      float scale, DistanceBias bias, void* out, hipStream_t stream) {
-#define SOMI_TILE_AS(DD, QB, KS_, BIAS)                                                                                 \
-    return launch_tile<DD, QB, KS_, BIAS>(q, q_stride, kc, vc, block_table, max_blocks, entry_start, entry_first_pos,    \
+                      float scale, DistanceBias bias, ScoreShape score, void* out, hipStream_t stream) {
+#define SOMI_TILE_AS(DD, QB, KS_, FORM)                                                                                 \
+    return launch_tile<DD, QB, KS_, FORM>(q, q_stride, kc, vc, block_table, max_blocks, entry_start, entry_first_pos,    \
                                           entry_len, n_entries, max_entry_len, nq, nkv, page_size, window, scale, bias, \
-                                          out, stream)
-#define SOMI_TILE(DD, QB, KS_)                                \
-    do {                                                      \
-        if (bias.length > 0) SOMI_TILE_AS(DD, QB, KS_, true); \
-        SOMI_TILE_AS(DD, QB, KS_, false);                     \
+                                          score, out, stream)
+#define SOMI_TILE(DD, QB, KS_)                                        \
+    do {                                                              \
+        if (bias.length > 0) SOMI_TILE_AS(DD, QB, KS_, SCORE_BIAS);   \
+        if (score.any()) SOMI_TILE_AS(DD, QB, KS_, SCORE_SHAPED);     \
+        SOMI_TILE_AS(DD, QB, KS_, SCORE_PLAIN);                       \
     } while (0)
     if (D == 128 && wide) SOMI_TILE(128, 8, 1);
     if (D == 128) SOMI_TILE(128, 4, 2);

@@ -4,8 +4,9 @@
 //   route      z = W_r h (float32), s = softmax(z) or, element by element, sigmoid(z); experts come in `groups` equal
 //              runs of neighbours, a run scores as its best expert and only the `keep` best runs stay; of their experts
 //              the `top` with the largest s are chosen, weighted by s over the chosen scores' sum (+ 1e-20) or by s as
-//              it is.  With a `correction` per expert the choice looks at s + correction, the weights at s alone.  Ties go
-//              to the lower index.
+//              it is.  With a `correction` per expert the choice looks at s + correction, the weights at s alone; a `bias`
+//              per expert is part of z itself.  Ties go to the lower index.  The router may hold one row more than there are
+//              experts: sigmoid of that row's product is the token's gate on the shared expert.
 //   align      the N * top pairs sorted by expert: order[], the experts' offsets and a list of row tiles
 //              (expert, first sorted row, rows) that the products' grids walk.
 //   gate_up    act[p, :] = glu(W_gate[e] h_t, W_up[e] h_t) for the sorted pair p = (t, e); where the pair's weight is to
@@ -13,7 +14,8 @@
 //   up         the same for experts without a gate: act[p, :] = relu(W_up[e] h_t)^2
 //   down       y[pair, :] = w_pair * (W_down[e] act[p, :]) (or without the weight), float32, at the pair's own place
 //              t * top + j
-//   combine    out[t, :] = sum_j y[t * top + j, :] (+ shared[t, :]), float32, in the order of j
+//   combine    out[t, :] = sum_j y[t * top + j, :] (+ shared[t, :], times the token's gate if there is one), float32, in
+//              the order of j
 //
 // glu(g, u) = g' sigmoid(alpha g') (u' + shift) with g' = min(g, limit) and u' = clamp(u, -limit, limit).
 // A row's sums run over K in one fixed order whatever else is in the batch.
@@ -138,22 +140,23 @@ __device__ __forceinline__ void wave_best(float& value, int& index) {
 template <typename T>
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __restrict__ router,
-                 const float* __restrict__ logits, const float* __restrict__ correction, int width, int experts,
-                 int top, int groups, int keep, int sigmoid_scores, int normalize, int* __restrict__ chosen,
-                 float* __restrict__ weight) {
+                 const float* __restrict__ logits, const float* __restrict__ bias, const float* __restrict__ correction,
+                 int width, int experts, int top, int groups, int keep, int sigmoid_scores, int normalize,
+                 int* __restrict__ chosen, float* __restrict__ weight, float* __restrict__ gate) {
     constexpr int PER_LANE = MOE_MAX_EXPERTS / 64;
-    __shared__ float score[MOE_MAX_EXPERTS];
+    __shared__ float score[MOE_MAX_EXPERTS + 1];
     __shared__ float pure[MOE_MAX_EXPERTS];         // the scores before the correction: what the weights are made of
     __shared__ int taken[MOE_MAX_EXPERTS];          // per run: kept or not
     __shared__ float pick_score[MOE_MAX_TOP];
     __shared__ int pick_index[MOE_MAX_TOP];
     const int64_t t = blockIdx.x;
     const int lane = threadIdx.x;
+    const int rows = experts + (gate != nullptr ? 1 : 0);      // of the router: the experts', then the gate's
     if (logits != nullptr) {
-        for (int e = lane; e < experts; e += 64) score[e] = logits[t * experts + e];
+        for (int e = lane; e < rows; e += 64) score[e] = logits[t * rows + e];
     } else {
         const T* row = x + t * row_stride;
-        for (int e = 0; e < experts; ++e) {
+        for (int e = 0; e < rows; ++e) {
             const float* w = router + (int64_t)e * width;
             float acc = 0.f;
             for (int i = lane; i < width; i += 64) acc += to_float(row[i]) * w[i];
@@ -167,10 +170,11 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
 #pragma unroll
     for (int j = 0; j < PER_LANE; ++j) {
         const int e = lane + 64 * j;
-        s[j] = e < experts ? score[e] : -INFINITY;
+        s[j] = e < experts ? score[e] + (bias != nullptr ? bias[e] : 0.f) : -INFINITY;
         top_z = fmaxf(top_z, s[j]);
     }
     top_z = wave_max(top_z);
+    if (gate != nullptr && lane == 0) gate[t] = 1.0f / (1.0f + expf(-score[experts]));
     float total = 0.f;
 #pragma unroll
     for (int j = 0; j < PER_LANE; ++j) {
@@ -260,9 +264,9 @@ moe_route_kernel(const T* __restrict__ x, int64_t row_stride, const float* __res
     }
 }
 
-extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, const float* router, const float* correction,
-                              float* logits, int n_tokens, int width, int experts, int top, int groups, int keep, int sigmoid_scores,
-                              int normalize, int* chosen, float* weight, hipStream_t stream) {
+extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, const float* router, const float* bias,
+                              const float* correction, float* logits, int n_tokens, int width, int experts, int top, int groups,
+                              int keep, int sigmoid_scores, int normalize, int* chosen, float* weight, float* gate, hipStream_t stream) {
     SOMI_REQUIRE(n_tokens >= 0 && width > 0 && experts > 0 && experts <= MOE_MAX_EXPERTS, "moe_route: %d experts, 1 to %d are supported",
                  experts, MOE_MAX_EXPERTS);
     SOMI_REQUIRE(groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups, "moe_route: %d groups (keep %d) do not divide %d experts",
@@ -270,15 +274,16 @@ extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, cons
     SOMI_REQUIRE(top >= 1 && top <= MOE_MAX_TOP && top <= keep * (experts / groups), "moe_route: top %d does not fit the kept experts", top);
     if (n_tokens == 0) return 0;
     SOMI_REQUIRE(dtype == SOMI_F32 || dtype == SOMI_BF16, "moe_route: unknown dtype %d", dtype);
-    // logits: a workspace [n_tokens, experts]; used where the tiled kernel applies (a width that is a multiple of 4)
+    // logits: a workspace [n_tokens, the router's rows]; used where the tiled kernel applies (a width that is a multiple of 4)
     const bool tiled = logits != nullptr && width % 4 == 0 && (uintptr_t)router % 16 == 0;
     if (tiled) {
-        const dim3 grid(ceil_div(n_tokens, ROUTE_TOKENS), ceil_div(experts, ROUTE_EXPERTS));
+        const int rows = experts + (gate != nullptr ? 1 : 0);
+        const dim3 grid(ceil_div(n_tokens, ROUTE_TOKENS), ceil_div(rows, ROUTE_EXPERTS));
         const int piece = dtype == SOMI_F32 ? 4 : 8;
         const bool wide = width % piece == 0 && row_stride % piece == 0 && (uintptr_t)x % 16 == 0;
 #define SOMI_ROUTE(T, W)                                                                                                  \
     hipLaunchKernelGGL((moe_router_logits_kernel<T, W>), grid, dim3(256), 0, stream, (const T*)x, row_stride, router, n_tokens, \
-                       width, experts, logits)
+                       width, rows, logits)
         if (dtype == SOMI_F32) {
             if (wide) SOMI_ROUTE(float, true); else SOMI_ROUTE(float, false);
         } else {
@@ -288,10 +293,12 @@ extern "C" int somi_moe_route(const void* x, int dtype, int64_t row_stride, cons
     }
     if (dtype == SOMI_F32)
         hipLaunchKernelGGL(moe_route_kernel<float>, dim3(n_tokens), dim3(64), 0, stream, (const float*)x, row_stride, router,
-                           tiled ? logits : nullptr, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
+                           tiled ? logits : nullptr, bias, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen,
+                           weight, gate);
     else
         hipLaunchKernelGGL(moe_route_kernel<bf16>, dim3(n_tokens), dim3(64), 0, stream, (const bf16*)x, row_stride, router,
-                           tiled ? logits : nullptr, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen, weight);
+                           tiled ? logits : nullptr, bias, correction, width, experts, top, groups, keep, sigmoid_scores, normalize, chosen,
+                           weight, gate);
     SOMI_LAUNCH_CHECK("moe_route");
     return 0;
 }
@@ -732,29 +739,30 @@ extern "C" int somi_moe_product_mfma(const void* a, int64_t a_stride, const void
 // out[t, :] = sum_j y[t * top + j, :] (+ shared[t, :]).
 template <typename T>
 __global__ void __launch_bounds__(256)
-moe_combine_kernel(const float* __restrict__ y, const T* __restrict__ shared_rows, int top, int width,
+moe_combine_kernel(const float* __restrict__ y, const T* __restrict__ shared_rows, const float* __restrict__ gate, int top, int width,
                    float* __restrict__ out) {
     const int64_t t = blockIdx.x;
     const int c = blockIdx.y * 256 + threadIdx.x;
     if (c >= width) return;
     float acc = 0.f;
     for (int j = 0; j < top; ++j) acc += y[(t * top + j) * width + c];
-    if (shared_rows != nullptr) acc += to_float(shared_rows[t * width + c]);
+    if (shared_rows != nullptr) acc = fmaf(to_float(shared_rows[t * width + c]), gate != nullptr ? gate[t] : 1.0f, acc);
     out[t * width + c] = acc;
 }
 
-extern "C" int somi_moe_combine(const float* y, const void* shared_rows, int shared_dtype, int n_tokens, int top, int width,
-                                float* out, hipStream_t stream) {
+// gate: [n_tokens], what multiplies a token's shared row, or null for 1.
+extern "C" int somi_moe_combine(const float* y, const void* shared_rows, int shared_dtype, const float* gate, int n_tokens, int top,
+                                int width, float* out, hipStream_t stream) {
     SOMI_REQUIRE(n_tokens >= 0 && top > 0 && width > 0, "moe_combine: bad sizes");
     if (n_tokens == 0) return 0;
     const dim3 grid(n_tokens, ceil_div(width, 256));
     SOMI_REQUIRE(grid.y <= 65535, "moe_combine: rows too wide");
     if (shared_rows == nullptr || shared_dtype == SOMI_F32)
-        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, stream, y, (const float*)shared_rows, top,
-                           width, out);
+        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, stream, y, (const float*)shared_rows, gate,
+                           top, width, out);
     else if (shared_dtype == SOMI_BF16)
-        hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, stream, y, (const bf16*)shared_rows, top,
-                           width, out);
+        hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, stream, y, (const bf16*)shared_rows, gate,
+                           top, width, out);
     else
         return somi_fail("moe_combine: unknown dtype %d", shared_dtype);
     SOMI_LAUNCH_CHECK("moe_combine");

@@ -145,3 +145,88 @@ extern "C" int somi_residual_add(float* h, const void* delta, int dtype, int64_t
     SOMI_LAUNCH_CHECK("residual_add");
     return 0;
 }
+
+// A sublayer's output joins the stream, and the sum is normed: h <- rmsnorm(alpha h + ls * y) * w, in place, with ls one
+// factor a channel.  COPY: the new rows also leave in TO.  V neighbouring values at a time, HELD of them kept by a thread;
+// a row of more than 256 * V * HELD values is read again for the scaling.
+template <typename TY, typename TO, bool COPY, int V, int HELD>
+__global__ void __launch_bounds__(256)
+join_norm_kernel(float* __restrict__ h, const TY* __restrict__ y, const float* __restrict__ ls, float alpha,
+                 const float* __restrict__ w, float eps, TO* __restrict__ copy, int width) {
+    __shared__ float red[16];
+    typedef __attribute__((ext_vector_type(V))) float vec;
+    typedef __attribute__((ext_vector_type(V))) TY yvec;
+    typedef __attribute__((ext_vector_type(V))) TO ovec;
+    const int64_t row = (int64_t)blockIdx.x * width;
+    auto sum_at = [&](int i) {
+        const vec hv = *reinterpret_cast<const vec*>(h + row + i), lv = *reinterpret_cast<const vec*>(ls + i);
+        const yvec yv = *reinterpret_cast<const yvec*>(y + row + i);
+        vec v;
+#pragma unroll
+        for (int x = 0; x < V; ++x) v[x] = fmaf(alpha, hv[x], lv[x] * to_float(yv[x]));
+        return v;
+    };
+    vec held[HELD];
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < HELD; ++c) {
+        const int i = (c * 256 + threadIdx.x) * V;
+        held[c] = 0.f;
+        if (i < width) held[c] = sum_at(i);
+#pragma unroll
+        for (int x = 0; x < V; ++x) ss = fmaf(held[c][x], held[c][x], ss);
+    }
+    for (int i = (HELD * 256 + threadIdx.x) * V; i < width; i += 256 * V) {
+        const vec v = sum_at(i);
+#pragma unroll
+        for (int x = 0; x < V; ++x) ss = fmaf(v[x], v[x], ss);
+    }
+    ss = block_sum<256>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)width + eps);
+    auto store = [&](int i, vec v) {
+        v *= inv * *reinterpret_cast<const vec*>(w + i);
+        *reinterpret_cast<vec*>(h + row + i) = v;
+        if (COPY) {
+            ovec o;
+#pragma unroll
+            for (int x = 0; x < V; ++x) o[x] = from_float<TO>(v[x]);
+            *reinterpret_cast<ovec*>(copy + row + i) = o;
+        }
+    };
+#pragma unroll
+    for (int c = 0; c < HELD; ++c) {
+        const int i = (c * 256 + threadIdx.x) * V;
+        if (i < width) store(i, held[c]);
+    }
+    for (int i = (HELD * 256 + threadIdx.x) * V; i < width; i += 256 * V) store(i, sum_at(i));
+}
+
+// h: [n, width] float32, updated in place; y: [n, width] of y_dtype; ls, w: [width] float32; copy: [n, width] bfloat16 or null.
+extern "C" int somi_join_norm(float* h, const void* y, int y_dtype, const float* ls, float alpha, const float* w, float eps,
+                              void* copy, int n, int width, hipStream_t stream) {
+    SOMI_REQUIRE(n >= 0 && width > 0, "join_norm: bad sizes n=%d width=%d", n, width);
+    SOMI_REQUIRE(eps >= 0.f, "join_norm: eps must be >= 0, got %g", (double)eps);
+    SOMI_REQUIRE(y_dtype == SOMI_F32 || y_dtype == SOMI_BF16, "join_norm: unknown dtype %d", y_dtype);
+    if (n == 0) return 0;
+    const bool vec = width % 4 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)ls % 16 == 0 &&
+                     (uintptr_t)w % 16 == 0 && (uintptr_t)copy % 16 == 0;
+#define SOMI_JOIN(TY, COPY, V, HELD)                                                                                      \
+    hipLaunchKernelGGL((join_norm_kernel<TY, bf16, COPY, V, HELD>), dim3(n), dim3(256), 0, stream, h, (const TY*)y, ls, alpha, \
+                       w, eps, (bf16*)copy, width)
+#define SOMI_JOIN_AS(TY, COPY)                                   \
+    do {                                                         \
+        if (!vec) SOMI_JOIN(TY, COPY, 1, 4);                     \
+        else if (width <= 1024) SOMI_JOIN(TY, COPY, 4, 1);       \
+        else if (width <= 2048) SOMI_JOIN(TY, COPY, 4, 2);       \
+        else SOMI_JOIN(TY, COPY, 4, 4);                          \
+    } while (0)
+    if (y_dtype == SOMI_F32) {
+        if (copy) SOMI_JOIN_AS(float, true); else SOMI_JOIN_AS(float, false);
+    } else {
+        if (copy) SOMI_JOIN_AS(bf16, true); else SOMI_JOIN_AS(bf16, false);
+    }
+#undef SOMI_JOIN_AS
+#undef SOMI_JOIN
+    SOMI_LAUNCH_CHECK("join_norm");
+    return 0;
+}

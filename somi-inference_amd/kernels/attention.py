@@ -45,25 +45,31 @@ def mfma_attention_supported(q: torch.Tensor, k_cache: torch.Tensor) -> bool:
             and q.data_ptr() % 16 == 0 and (q.shape[1] * 2) % 16 == 0)
 
 
-def bias_supported(k_cache: torch.Tensor, block_table: torch.Tensor) -> bool:
-    """The matrix-core kernels take a distance bias at these sizes (head sizes 32 to 128, pages of a power of two keys)."""
+def forms_supported(k_cache: torch.Tensor, block_table: torch.Tensor) -> bool:
+    """The matrix-core kernels take a distance bias, or capped, chunked and sinking scores, at these sizes (head sizes 32
+    to 128, pages of a power of two keys)."""
     return bool(ops.library().somi_attention_bias_supported(k_cache.shape[3], k_cache.shape[2], block_table.shape[1]))
 
 
 def paged_attention(qkv: torch.Tensor, num_heads: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
                     block_table: torch.Tensor, step, *, window: int, scale: float,
-                    bias: torch.Tensor | None = None) -> torch.Tensor:
+                    bias: torch.Tensor | None = None, score: "ops.ScoreShape | None" = None) -> torch.Tensor:
     """Attention of every token of the step over its request's cache pages -> [N, nq * D].
 
     ``qkv`` holds each token's query heads first in its row (rotated already).  float32, and shapes the
     MFMA kernels do not take (head sizes that are no multiple of 16, page sizes that are no multiple
     of 4), run the plain kernel.  ``bias``: [heads, length] float32 added to the scaled scores by distance (its last
-    entry is 0 and stands for every key farther back).
+    entry is 0 and stands for every key farther back).  ``score``: a cap, chunks, a sink (:class:`ops.ScoreShape`).
     """
-    if not mfma_attention_supported(qkv, k_cache) or (bias is not None and not bias_supported(k_cache, block_table)):
+    if score is not None and not score.any:
+        score = None
+    if not mfma_attention_supported(qkv, k_cache) or ((bias is not None or score is not None)
+                                                      and not forms_supported(k_cache, block_table)):
         return ops.paged_attention_plain(qkv, qkv.shape[1], k_cache, v_cache, block_table,
-                                         step.token_entry, step.positions, num_heads, window, scale, bias)
+                                         step.token_entry, step.positions, num_heads, window, scale, bias, score)
     nkv, head_dim = k_cache.shape[1], k_cache.shape[3]
+    # what a decoded token sees at most: with chunks, its own (whose first key may lie inside a 32-key tile)
+    context = min(step.max_context, score.chunk + 32) if score is not None and score.chunk else step.max_context
     groups = nkv * ((num_heads // nkv + 15) // 16)
     out = torch.empty((qkv.shape[0], num_heads * head_dim), dtype=qkv.dtype, device=qkv.device)
     if step.max_entry_len > DECODE_PORTION:
@@ -77,13 +83,15 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, k_cache: torch.Tensor, v_
                              f"of its {step.num_tokens} tokens: rows of the output would stay unwritten")
         ops.attention_prefill(qkv, qkv.shape[1], k_cache, v_cache, block_table, step.entry_start,
                               step.entry_first_position, step.max_entry_len, num_heads, window, scale, out,
-                              max_context=step.max_context, entry_len=split.long_entry_len if short else None, bias=bias)
+                              max_context=step.max_context, entry_len=split.long_entry_len if short else None, bias=bias,
+                              score=score)
         if short:
-            split_len, num_splits = decode_splits(short, groups, step.max_context, k_cache.shape[2], head_dim)
+            split_len, num_splits = decode_splits(short, groups, context, k_cache.shape[2], head_dim)
             ops.attention_decode(qkv, qkv.shape[1], k_cache, v_cache, block_table, step.token_entry, step.positions,
-                                 num_heads, window, scale, split_len, num_splits, out, token_list=split.short_tokens, bias=bias)
+                                 num_heads, window, scale, split_len, num_splits, out, token_list=split.short_tokens, bias=bias,
+                                 score=score)
         return out
-    split_len, num_splits = decode_splits(step.num_tokens, groups, step.max_context, k_cache.shape[2], head_dim)
+    split_len, num_splits = decode_splits(step.num_tokens, groups, context, k_cache.shape[2], head_dim)
     ops.attention_decode(qkv, qkv.shape[1], k_cache, v_cache, block_table, step.token_entry, step.positions,
-                         num_heads, window, scale, split_len, num_splits, out, bias=bias)
+                         num_heads, window, scale, split_len, num_splits, out, bias=bias, score=score)
     return out

@@ -10,6 +10,7 @@ when the extension cannot be built or loaded.
 from __future__ import annotations
 
 import ctypes
+from typing import NamedTuple
 
 import torch
 
@@ -134,6 +135,21 @@ def rmsnorm(h: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.
     return out
 
 
+def join_norm(h: torch.Tensor, y: torch.Tensor, scale: torch.Tensor, alpha: float, weight: torch.Tensor, eps: float,
+              copy: bool) -> torch.Tensor | None:
+    """h <- rmsnorm(alpha h + scale * y) * weight in place, float32; y: rows in either type; scale: one factor a channel.
+    ``copy``: the new rows in bfloat16 are returned."""
+    _need(h, "residual stream", torch.float32)
+    n, width = h.shape
+    _need(y, "sublayer rows", None, (n, width))
+    _need(scale, "sublayer scale", torch.float32, (width,))
+    _need(weight, "norm weight", torch.float32, (width,))
+    out = torch.empty((n, width), dtype=torch.bfloat16, device=h.device) if copy else None
+    _check(library().somi_join_norm(_ptr(h), _ptr(y), dtype_code(y.dtype), _ptr(scale), ctypes.c_float(alpha), _ptr(weight),
+                                    ctypes.c_float(eps), _ptr(out), n, width, _stream()))
+    return out
+
+
 def residual_add(h: torch.Tensor, delta: torch.Tensor) -> None:
     _need(h, "residual stream", torch.float32)
     _need(delta, "residual delta", None, tuple(h.shape))
@@ -218,9 +234,32 @@ def _bias_arguments(bias: torch.Tensor | None, heads: int) -> tuple[ctypes.c_voi
     return _ptr(bias), bias.shape[1]
 
 
+class ScoreShape(NamedTuple):
+    """What is done to attention scores beside the scale and a causal mask or window: ``softcap`` c turns a scaled score s
+    into c tanh(s / c); with ``chunk`` n a query sees only keys of its own run of n positions, counted from the sequence's
+    start; ``sink`` [heads] float32 puts exp(sink) into the softmax's denominator."""
+
+    softcap: float | None = None
+    chunk: int | None = None
+    sink: torch.Tensor | None = None
+
+    @property
+    def any(self) -> bool:
+        return bool(self.softcap) or bool(self.chunk) or self.sink is not None
+
+
+def _score_arguments(shape: ScoreShape | None, heads: int) -> tuple[ctypes.c_float, int, ctypes.c_void_p]:
+    if shape is None:
+        return ctypes.c_float(0.0), 0, _ptr(None)
+    if shape.sink is not None:
+        _need(shape.sink, "attention sink", torch.float32, (heads,))
+    return ctypes.c_float(shape.softcap or 0.0), int(shape.chunk or 0), _ptr(shape.sink)
+
+
 def paged_attention_plain(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
                           block_table: torch.Tensor, token_entry: torch.Tensor, positions: torch.Tensor,
-                          nq: int, window: int, scale: float, bias: torch.Tensor | None = None) -> torch.Tensor:
+                          nq: int, window: int, scale: float, bias: torch.Tensor | None = None,
+                          shape: ScoreShape | None = None) -> torch.Tensor:
     """Causal attention of every token over its request's cached keys (plain float32 kernel).
 
     q: a tensor whose row t holds the nq query heads of token t first (row stride q_stride elements).  ``bias``: a
@@ -242,7 +281,7 @@ def paged_attention_plain(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor,
     _check(library().somi_paged_attention_plain(
         _ptr(q), dtype_code(q.dtype), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table),
         block_table.shape[1], _ptr(token_entry), _ptr(positions), n, nq, nkv, head_dim, page_size, window,
-        ctypes.c_float(scale), *_bias_arguments(bias, nq), _ptr(out), _stream()))
+        ctypes.c_float(scale), *_bias_arguments(bias, nq), *_score_arguments(shape, nq), _ptr(out), _stream()))
     return out
 
 
@@ -250,7 +289,7 @@ def attention_decode(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_ca
                      block_table: torch.Tensor, token_entry: torch.Tensor, positions: torch.Tensor,
                      nq: int, window: int, scale: float, split_len: int, num_splits: int,
                      out: torch.Tensor, token_list: torch.Tensor | None = None,
-                     bias: torch.Tensor | None = None) -> None:
+                     bias: torch.Tensor | None = None, score: ScoreShape | None = None) -> None:
     """MFMA attention of the listed tokens (all when ``token_list`` is None) over their pages, written
     into ``out`` ([N, nq * D] bfloat16).  The keys of a request are cut into ``num_splits`` ranges of
     ``split_len`` positions that run in parallel and are merged afterwards."""
@@ -278,7 +317,7 @@ def attention_decode(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_ca
     _check(library().somi_attention_decode(
         _ptr(q), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
         _ptr(token_list), _ptr(token_entry), _ptr(positions), n_list, nq, nkv, head_dim, page_size, window,
-        ctypes.c_float(scale), split_len, num_splits, *_bias_arguments(bias, nq), _ptr(out), _ptr(part_acc), _ptr(part_ml),
+        ctypes.c_float(scale), split_len, num_splits, *_bias_arguments(bias, nq), *_score_arguments(score, nq), _ptr(out), _ptr(part_acc), _ptr(part_ml),
         _stream()))
 
 
@@ -286,7 +325,7 @@ def attention_prefill(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_c
                       block_table: torch.Tensor, entry_start: torch.Tensor, entry_first_position: torch.Tensor,
                       max_entry_len: int, nq: int, window: int, scale: float, out: torch.Tensor,
                       max_context: int = 0, shape: int = 0, entry_len: torch.Tensor | None = None,
-                      bias: torch.Tensor | None = None) -> None:
+                      bias: torch.Tensor | None = None, score: ScoreShape | None = None) -> None:
     """MFMA causal attention of every token of every portion over its request's pages, into ``out``
     ([N, nq * D] bfloat16).  entry_start: [E + 1] int32 offsets of the portions in the flat batch;
     entry_first_position: [E] int32.  ``max_context``: the longest context a portion ends at, a hint for the
@@ -317,7 +356,8 @@ def attention_prefill(q: torch.Tensor, q_stride: int, k_cache: torch.Tensor, v_c
     _check(library().somi_attention_prefill(
         _ptr(q), ctypes.c_int64(q_stride), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
         _ptr(entry_start), _ptr(entry_first_position), _ptr(entry_len), entries, max_entry_len, max(0, int(max_context)), int(shape), nq, nkv,
-        head_dim, page_size, window, ctypes.c_float(scale), *_bias_arguments(bias, nq), _ptr(out), _stream()))
+        head_dim, page_size, window, ctypes.c_float(scale), *_bias_arguments(bias, nq), *_score_arguments(score, nq), _ptr(out),
+        _stream()))
 
 
 def silu_mul(gate_up: torch.Tensor, block: int = 0) -> torch.Tensor:
@@ -1064,6 +1104,36 @@ def qk_norm_store(rows: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tenso
 
 
 # ------------------------------------------------------------------------------------------ the gated delta rule
+def qk_norm_rope_store(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tensor,
+                       k_weight: torch.Tensor, eps: float, inv_freq: torch.Tensor | None, rotary_dim: int, heads: int,
+                       kv_heads: int, dim: int, vdim: int, k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
+    """From rows [q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim)]: q and k RMS-normed over their whole
+    projections, the first ``rotary_dim`` channels of their heads turned (channel j with j + rotary_dim / 2, by position *
+    inv_freq[j]); k and v into the tokens' slots of ``k_cache`` [pages, kv_heads, page, padded] and ``v_cache`` [pages,
+    kv_heads, padded, page] -> q [N, heads * padded] in the caches' dtype.  Channels past dim and vdim are zeros."""
+    _need(rows, "projected rows")
+    n = rows.shape[0]
+    if rows.shape[1] < (heads + kv_heads) * dim + kv_heads * vdim:
+        raise KernelError(f"qk_norm_rope_store: rows of {rows.shape[1]} values do not hold the projections")
+    _need(k_cache, "key pages")
+    if k_cache.dim() != 4 or k_cache.shape[1] != kv_heads:
+        raise KernelError(f"qk_norm_rope_store: key pages {tuple(k_cache.shape)} != [pages, {kv_heads}, page, padded]")
+    page, padded = k_cache.shape[2], k_cache.shape[3]
+    _need(v_cache, "value pages", k_cache.dtype, _v_shape(k_cache))
+    _need(positions, "positions", torch.int32, (n,))
+    _need(slots, "slot mapping", torch.int32, (n,))
+    _need(q_weight, "q norm weight", torch.float32, (heads * dim,))
+    _need(k_weight, "k norm weight", torch.float32, (kv_heads * dim,))
+    if inv_freq is not None:
+        _need(inv_freq, "inv_freq", torch.float32, (rotary_dim // 2,))
+    q = torch.empty((n, heads * padded), dtype=k_cache.dtype, device=rows.device)
+    _check(library().somi_qk_norm_rope_store(_ptr(rows), dtype_code(rows.dtype), ctypes.c_int64(rows.shape[1]), _ptr(positions),
+                                             _ptr(slots), _ptr(q_weight), _ptr(k_weight), ctypes.c_float(eps), _ptr(inv_freq),
+                                             int(rotary_dim), n, int(heads), int(kv_heads), int(dim), int(vdim), padded, _ptr(q),
+                                             _ptr(k_cache), _ptr(v_cache), page, dtype_code(k_cache.dtype), _stream()))
+    return q
+
+
 SHORT_CONV_MAX_TAPS = 9
 
 
@@ -1182,11 +1252,13 @@ ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, groups: int, keep: int, scores: str = "softmax",
-              normalize: bool = True, correction: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+              normalize: bool = True, correction: torch.Tensor | None = None, bias: torch.Tensor | None = None,
+              gate: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """Chosen experts [N, top] int32 and their weights [N, top] float32: float32 scores (``scores``: the softmax over all
     experts, or each expert's own sigmoid), the ``keep`` best of ``groups`` runs of neighbouring experts, the ``top`` best
     experts of those; weights over their sum (``normalize``) or the scores as they are.  ``correction`` [experts] float32 is
-    added to the scores for the choice, not for the weights."""
+    added to the scores for the choice, not for the weights; ``bias`` [experts] float32 to the router's sums.  ``gate`` [N]
+    float32: the router's last row is no expert's, the sigmoid of its sum goes there."""
     _need(x, "rows")
     n, width = x.shape
     _need(router, "router", torch.float32)
@@ -1194,15 +1266,19 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, top: int, groups: int, keep
         raise KernelError(f"moe_route: router {tuple(router.shape)} does not fit rows of {width}")
     if scores not in ROUTER_SCORES:
         raise KernelError(f"moe_route: unknown scores {scores!r}; known: {sorted(ROUTER_SCORES)}")
+    experts = router.shape[0] - (1 if gate is not None else 0)
     if correction is not None:
-        _need(correction, "choice correction", torch.float32, (router.shape[0],))
+        _need(correction, "choice correction", torch.float32, (experts,))
+    if bias is not None:
+        _need(bias, "router bias", torch.float32, (experts,))
+    if gate is not None:
+        _need(gate, "shared expert's gate", torch.float32, (n,))
     chosen = torch.empty((n, top), dtype=torch.int32, device=x.device)
     weight = torch.empty((n, top), dtype=torch.float32, device=x.device)
     logits = torch.empty((n, router.shape[0]), dtype=torch.float32, device=x.device)     # the router's sums, if it tiles them
-    _check(library().somi_moe_route(_ptr(x), dtype_code(x.dtype), ctypes.c_int64(x.stride(0)), _ptr(router), _ptr(correction),
-                                    _ptr(logits), n,
-                                    width, router.shape[0], int(top), int(groups), int(keep), ROUTER_SCORES[scores],
-                                    1 if normalize else 0, _ptr(chosen), _ptr(weight), _stream()))
+    _check(library().somi_moe_route(_ptr(x), dtype_code(x.dtype), ctypes.c_int64(x.stride(0)), _ptr(router), _ptr(bias),
+                                    _ptr(correction), _ptr(logits), n, width, experts, int(top), int(groups), int(keep),
+                                    ROUTER_SCORES[scores], 1 if normalize else 0, _ptr(chosen), _ptr(weight), _ptr(gate), _stream()))
     return chosen, weight
 
 
@@ -1301,16 +1377,18 @@ def moe_down(act: torch.Tensor, down: torch.Tensor, tiles: torch.Tensor, order: 
     return y
 
 
-def moe_combine(y: torch.Tensor, top: int, shared: torch.Tensor | None) -> torch.Tensor:
-    """out[t] = sum_j y[t * top + j] (+ shared[t]) -> [N, width] float32."""
+def moe_combine(y: torch.Tensor, top: int, shared: torch.Tensor | None, gate: torch.Tensor | None = None) -> torch.Tensor:
+    """out[t] = sum_j y[t * top + j] (+ shared[t], times gate[t] if there is one) -> [N, width] float32."""
     _need(y, "expert outputs", torch.float32)
     pairs, width = y.shape
     n = pairs // top
     if shared is not None:
         _need(shared, "shared expert rows", None, (n, width))
+    if gate is not None:
+        _need(gate, "shared expert's gate", torch.float32, (n,))
     out = torch.empty((n, width), dtype=torch.float32, device=y.device)
-    _check(library().somi_moe_combine(_ptr(y), _ptr(shared), dtype_code(shared.dtype) if shared is not None else 0, n, int(top),
-                                      width, _ptr(out), _stream()))
+    _check(library().somi_moe_combine(_ptr(y), _ptr(shared), dtype_code(shared.dtype) if shared is not None else 0, _ptr(gate), n,
+                                      int(top), width, _ptr(out), _stream()))
     return out
 
 
@@ -1774,6 +1852,9 @@ def _float_rows(t: torch.Tensor, n: int, width: int, name: str) -> ctypes.c_int6
     return ctypes.c_int64(t.stride(0))
 
 
+SSD_MAX_ROWS = 512           # rows of a head's state
+
+
 def ssd_chunked(p: int, n_state: int) -> bool:
     """The chunked kernels take heads of ``p`` channels with a state of ``n_state`` rows."""
     return bool(library().somi_ssd_chunked(int(p), int(n_state)))
@@ -1819,6 +1900,82 @@ def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, gro
                                            _rows_out(out, n, width, "gated_group_norm"), dtype_code(out.dtype), _stream()))
 
 
+def ssd_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, step, state: torch.Tensor, *, keep: torch.Tensor,
+               write: torch.Tensor | None = None, scale: float = 1.0,
+               chunked: bool = True) -> tuple[torch.Tensor, torch.Tensor | None]:
+    """S <- a S + w k v^T; y = scale S^T q per head -> (y [N, heads * P] float32, the normaliser's products or None).
+    q, k: [N, heads * D], v: [N, heads * P], float32 columns of rows of one stride.  With ``write``: keep and write are a
+    and w, [N, heads], and the head also keeps n <- a n + w k and gives scale n . q, [N, heads]; without: keep holds the
+    heads' fixed decays, [heads], and w is 1.  state: [slots, heads, P (+ 1), D] float32, read and written in place, the
+    normaliser last.  ``chunked`` as in :func:`ssd`."""
+    _need(state, "recurrent state", torch.float32)
+    _, heads, rows, d = state.shape
+    p = rows - (1 if write is not None else 0)
+    n = q.shape[0]
+    strides = {_float_rows(q, n, heads * d, "queries").value, _float_rows(k, n, heads * d, "keys").value,
+               _float_rows(v, n, heads * p, "values").value}
+    if len(strides) != 1:
+        raise KernelError(f"ssd_memory: queries, keys and values must be columns of the same rows, got strides {sorted(strides)}")
+    stride = strides.pop()
+    for t, name in ((keep, "decays"), (write, "write weights")):
+        if t is not None:
+            _need(t, name, torch.float32, (n, heads) if write is not None else (heads,))
+    entries = step.state_slots.numel()
+    _need(step.entry_start, "entry offsets", torch.int32, (entries + 1,))
+    _need(step.state_slots, "state slots", torch.int32, (entries,))
+    y = torch.empty((n, heads * p), dtype=torch.float32, device=q.device)
+    den = torch.empty((n, heads), dtype=torch.float32, device=q.device) if write is not None else None
+    local = decay = None
+    aligned = stride % 4 == 0 and all(t.data_ptr() % 16 == 0 for t in (q, k, v))
+    if chunked and aligned and step.max_entry_len >= library().somi_ssd_chunked_from() and ssd_chunked(p, d):
+        chunks = library().somi_ssd_chunks(n, entries)
+        local = torch.empty((chunks, heads, rows, d), dtype=torch.float32, device=q.device)
+        decay = torch.empty((chunks, heads), dtype=torch.float32, device=q.device)
+    _check(library().somi_ssd_memory(_ptr(q), _ptr(k), _ptr(v), ctypes.c_int64(stride), _ptr(keep), _ptr(write), ctypes.c_float(scale),
+                                     _ptr(step.entry_start), _ptr(step.state_slots), _ptr(state), entries, int(step.max_entry_len),
+                                     heads, p, d, _ptr(local), _ptr(decay), _ptr(y), _ptr(den), _stream()))
+    return y, den
+
+
+def mlstm_gates(rows_i: torch.Tensor, rows_f: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, cap: float, step,
+                top: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
+    """(keep, write, floor), each [N, heads] float32, from the gates' projections [N, heads] (float32, columns of rows of one
+    stride): i = cap tanh((ri + b_i) / cap), f = log sigmoid(cap tanh((rf + b_f) / cap)), m <- max(f + m, i); keep = exp(f +
+    m_before - m), write = exp(i - m), floor = exp(-m).  top: [slots, heads] float32, the maxima m, read and written."""
+    _need(top, "running maxima", torch.float32)
+    heads = top.shape[1]
+    n = rows_i.shape[0]
+    stride = _float_rows(rows_i, n, heads, "input gates")
+    if _float_rows(rows_f, n, heads, "forget gates").value != stride.value:
+        raise KernelError("mlstm_gates: both gates must be columns of the same rows")
+    _need(bias_i, "input gate bias", torch.float32, (heads,))
+    _need(bias_f, "forget gate bias", torch.float32, (heads,))
+    entries = step.state_slots.numel()
+    _need(step.entry_start, "entry offsets", torch.int32, (entries + 1,))
+    _need(step.state_slots, "state slots", torch.int32, (entries,))
+    keep, write, floor = (torch.empty((n, heads), dtype=torch.float32, device=top.device) for _ in range(3))
+    _check(library().somi_mlstm_gates(_ptr(rows_i), _ptr(rows_f), stride, _ptr(bias_i), _ptr(bias_f), ctypes.c_float(cap),
+                                      _ptr(step.entry_start), _ptr(step.state_slots), _ptr(top), entries, int(step.max_entry_len),
+                                      heads, _ptr(keep), _ptr(write), _ptr(floor), _stream()))
+    return keep, write, floor
+
+
+def norm_sigmoid_gate(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, scale: float,
+                      out: torch.Tensor, den: torch.Tensor | None = None, floor: torch.Tensor | None = None) -> None:
+    """out = scale * weight * rms-normed(u) * sigmoid(gate), the root mean square over each of ``groups`` equal parts of a
+    row; u = y or, with ``den`` and ``floor`` [N, groups], y / (max(|den|, floor) + 1e-6).  y: [N, width] float32; gate:
+    float32, possibly columns of wider rows; out: [N, width], likewise."""
+    _need(y, "rows", torch.float32)
+    n, width = y.shape
+    _need(weight, "norm weight", torch.float32, (width,))
+    for t, name in ((den, "normaliser"), (floor, "normaliser's floor")):
+        if t is not None:
+            _need(t, name, torch.float32, (n, groups))
+    _check(library().somi_norm_sigmoid_gate(_ptr(y), _ptr(den), _ptr(floor), _ptr(gate), _float_rows(gate, n, width, "gate rows"),
+                                            _ptr(weight), int(groups), ctypes.c_float(eps), ctypes.c_float(scale), n, width,
+                                            _ptr(out), _rows_out(out, n, width, "norm_sigmoid_gate"), dtype_code(out.dtype), _stream()))
+
+
 def min_gru(rows: torch.Tensor, z_bias: torch.Tensor, x_bias: torch.Tensor, step, state: torch.Tensor, scale: float,
             out: torch.Tensor) -> None:
     """S <- (1 - z) S + z c element by element with z = sigmoid(rz + z_bias), u = rx + x_bias, c = u + 1/2 (u >= 0) or
@@ -1844,6 +2001,12 @@ def squared_relu(z: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
     out = torch.empty(z.shape, dtype=out_dtype, device=z.device)
     _check(library().somi_squared_relu(_ptr(z), _ptr(out), dtype_code(out_dtype), ctypes.c_int64(z.numel()), _stream()))
     return out
+
+
+def silu_columns_(rows: torch.Tensor) -> None:
+    """SiLU in place on float32 rows, possibly columns of wider rows."""
+    n, width = rows.shape
+    _check(library().somi_silu_columns(_ptr(rows), _float_rows(rows, n, width, "rows"), n, width, _stream()))
 
 
 def xielu(z: torch.Tensor, pq: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:

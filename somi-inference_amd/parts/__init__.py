@@ -4,7 +4,7 @@ from .attention import GroupedQueryAttention
 from .base import (PAGE, Block, BorrowedCache, CompositeSpec, FeedForward, FixedStateSpec, LayerCache, Mixer, Norm, PagedKVSpec, PagedSpec,
                    PageTensor, Part, PartSpec, PositionEncoding, Runtime)
 from .biased_attention import BiasedAttention
-from .block import HyperConnectionBlock, OutputNormBlock, ParallelBlock, PreNormBlock
+from .block import HyperConnectionBlock, OutputNormBlock, ParallelBlock, PreNormBlock, SumNormBlock
 from .delta_rule import GatedDeltaRule
 from .diff_attention import DifferentialAttention
 from .embedding import LMHead, TokenEmbedding
@@ -13,9 +13,11 @@ from .gla import GatedLinearAttention
 from .hgrn2 import HGRN2
 from .input_conv import ShortConvInput
 from .latent_attention import LatentAttention
+from .lightning import LightningAttention
 from .mamba2 import Mamba2
 from .min_gru import MinGRU
 from .mixed_attention import MixedHeadsAttention
+from .mlstm import MLSTM
 from .moe import RoutedExperts
 from .norm import DynamicTanh, LayerNorm, RMSNorm
 from .parallel_mixer import ParallelMixers
@@ -41,6 +43,8 @@ register_part("mixer", "mixed_heads_attention", MixedHeadsAttention)
 register_part("mixer", "biased_attention", BiasedAttention)
 register_part("mixer", "mamba2", Mamba2)
 register_part("mixer", "min_gru", MinGRU)
+register_part("mixer", "mlstm", MLSTM)
+register_part("mixer", "lightning_attention", LightningAttention)
 register_part("feed_forward", "swiglu", SwiGLU)
 register_part("feed_forward", "routed_experts", RoutedExperts)
 register_part("feed_forward", "poly_norm", PolyNormFF)
@@ -51,11 +55,12 @@ register_part("block", "pre_norm", PreNormBlock)
 register_part("block", "parallel", ParallelBlock)
 register_part("block", "output_norm", OutputNormBlock)
 register_part("block", "hyper_connections", HyperConnectionBlock)
+register_part("block", "sum_norm", SumNormBlock)
 register_part("embedding", "token_embedding", TokenEmbedding)
 register_part("head", "lm_head", LMHead)
 
 __all__ = [
-    "ActivatedFF", "BiasedAttention", "Mamba2", "MinGRU", "RowsMixer", "Block", "BorrowedCache", "HyperConnectionBlock", "MixedHeadsAttention", "CompositeSpec", "HGRN2", "LatentAttention", "LayerNorm", "OutputNormBlock", "PolyNormFF", "ShortConvInput", "DifferentialAttention", "DynamicTanh", "GatedDeltaRule", "GatedTokenInput", "ParallelBlock", "ParallelMixers", "RoutedExperts", "FeedForward", "FixedStateSpec", "GatedLinearAttention", "GroupedQueryAttention", "LMHead", "LayerCache", "Mixer",
+    "ActivatedFF", "BiasedAttention", "LightningAttention", "MLSTM", "SumNormBlock", "Mamba2", "MinGRU", "RowsMixer", "Block", "BorrowedCache", "HyperConnectionBlock", "MixedHeadsAttention", "CompositeSpec", "HGRN2", "LatentAttention", "LayerNorm", "OutputNormBlock", "PolyNormFF", "ShortConvInput", "DifferentialAttention", "DynamicTanh", "GatedDeltaRule", "GatedTokenInput", "ParallelBlock", "ParallelMixers", "RoutedExperts", "FeedForward", "FixedStateSpec", "GatedLinearAttention", "GroupedQueryAttention", "LMHead", "LayerCache", "Mixer",
     "NoPosition", "Norm", "PAGE", "PageTensor", "PagedKVSpec", "PagedSpec", "Part", "PartSpec", "PositionEncoding", "PreNormBlock", "RMSNorm",
     "ResidualStream", "RotaryPosition", "Runtime", "SwiGLU", "TokenEmbedding", "build_part", "part_kinds",
     "register_part", "unregister_part",

@@ -87,13 +87,15 @@ class PagedSpec:
     """Something kept for every past token, in pages: the tensors a page holds, how many of the latest tokens
     stay visible (``window``, the current one included; None = all), how many of a request's first tokens stay
     visible beside the window (``keep_first``), and the page size the mixer's kernels want (None = the engine's).
-    Layers whose window, kept tokens and page size agree share one pool of pages and one block table per request;
-    each layer run has its own tensors."""
+    ``chunk``: only the tokens of the current one's run of ``chunk`` positions, counted from a request's first token, stay
+    visible (None = no such runs).  Layers whose window, chunk, kept tokens and page size agree share one pool of pages and
+    one block table per request; each layer run has its own tensors."""
 
     tensors: tuple[PageTensor, ...]
     window: int | None = None
     page_size: int | None = None
     keep_first: int = 0
+    chunk: int | None = None
 
     def __post_init__(self) -> None:
         names = [t.name for t in self.tensors]
@@ -103,6 +105,8 @@ class PagedSpec:
             raise ValueError(f"page size {self.page_size} must be >= 1")
         if self.keep_first < 0 or (self.window is not None and self.window < 1):
             raise ValueError(f"a window must be >= 1 and kept tokens >= 0, got {self.window} and {self.keep_first}")
+        if self.chunk is not None and (self.chunk < 1 or self.keep_first):
+            raise ValueError(f"a chunk must be >= 1 and comes without kept first tokens, got {self.chunk} and {self.keep_first}")
 
 
 class PagedKVSpec(PagedSpec):
@@ -110,9 +114,10 @@ class PagedKVSpec(PagedSpec):
     page, ``[pages, kv_heads, head_dim, page]`` (consecutive positions of one channel are adjacent: the operand
     layout of the weights-times-values product)."""
 
-    def __init__(self, num_kv_heads: int, head_dim: int, window: int | None = None, page_size: int | None = None) -> None:
+    def __init__(self, num_kv_heads: int, head_dim: int, window: int | None = None, page_size: int | None = None,
+                 chunk: int | None = None) -> None:
         super().__init__((PageTensor("k", (int(num_kv_heads), PAGE, int(head_dim))),
-                          PageTensor("v", (int(num_kv_heads), int(head_dim), PAGE))), window, page_size)
+                          PageTensor("v", (int(num_kv_heads), int(head_dim), PAGE))), window, page_size, chunk=chunk)
         object.__setattr__(self, "num_kv_heads", int(num_kv_heads))
         object.__setattr__(self, "head_dim", int(head_dim))
 
@@ -240,6 +245,11 @@ class Norm(Part):
         """h += norm(y) in place on the float32 residual rows, for arrangements that norm a sublayer's output instead of
         its input; with ``copy_dtype`` the new rows are also returned in that dtype.  Norms that offer it override it."""
         raise NotImplementedError(f"{type(self).__name__} does not norm a sublayer's output")
+
+    def join_normed(self, h: torch.Tensor, y: torch.Tensor, scale: torch.Tensor, alpha: float) -> torch.Tensor:
+        """h <- norm(alpha h + scale * y) in place on the float32 residual rows (scale: one factor a channel), for
+        arrangements that norm the sum; the new rows are returned in the compute dtype.  Norms that offer it override it."""
+        raise NotImplementedError(f"{type(self).__name__} does not norm a sum")
 
 
 class PositionEncoding(Part):

@@ -162,6 +162,65 @@ class OutputNormBlock(Block):
             self.token_input.add_to(h, x, step, 1.0)
 
 
+class SumNormBlock(Block):
+    """The norm sits on the sum, and the sublayers read the stream itself:
+
+        h <- norm1(alpha h + s1 * mixer(h));     h <- norm2(alpha h + s2 * feed_forward(h))
+
+    with one factor a channel, s1 and s2 (the tensors ``scale1`` and ``scale2`` of ``names``; None there: no such tensor, a
+    factor of one).  The sum, the scaling and the norm are float32, done by one kernel that also leaves the new rows as the
+    next sublayer reads them; a sublayer's last product is computed into float32 rows.  The norms are any that offer
+    ``join_normed``.  A layer without a feed-forward has the first sublayer only.  ``names``: the sub-prefixes of the two
+    norms, the mixer and the feed-forward, and the two scales' names."""
+
+    DEFAULT_NAMES = {"mixer_norm": "norm1", "mixer": "mix", "ffn_norm": "norm2", "feed_forward": "mlp", "mixer_scale": "ls1",
+                     "ffn_scale": "ls2"}
+
+    def __init__(self, prefix: str, mixer: PartSpec, feed_forward: PartSpec | None, mixer_norm: PartSpec,
+                 ffn_norm: PartSpec | None = None, width: int = 0, alpha: float = 1.0,
+                 names: dict[str, str | None] | None = None) -> None:
+        super().__init__(prefix)
+        sub = dict(self.DEFAULT_NAMES)
+        sub.update(names or {})
+        self.sub, self.width, self.alpha = sub, int(width), float(alpha)
+        self.mixer_norm = build_part("norm", mixer_norm, prefix=self.name(sub["mixer_norm"]))
+        self.mixer = build_part("mixer", mixer, prefix=self.name(sub["mixer"]))
+        self.ffn_norm = self.feed_forward = None
+        if feed_forward is not None:
+            if ffn_norm is None:
+                raise ValueError(f"{prefix}: a feed-forward needs its norm")
+            self.ffn_norm = build_part("norm", ffn_norm, prefix=self.name(sub["ffn_norm"]))
+            self.feed_forward = build_part("feed_forward", feed_forward, prefix=self.name(sub["feed_forward"]))
+        self.graph_safe = all(getattr(part, "graph_safe", False) for part in self.parts())
+
+    def parts(self) -> list[Part]:
+        return [part for part in (self.mixer, self.mixer_norm, self.feed_forward, self.ffn_norm) if part is not None]
+
+    def _scales(self) -> list[str | None]:
+        roles = ["mixer_scale"] + (["ffn_scale"] if self.feed_forward is not None else [])
+        return [self.name(self.sub[role]) if self.sub[role] else None for role in roles]
+
+    def weight_specs(self):
+        return super().weight_specs() + [WeightSpec(name, (self.width,), VECTOR, Init(1.0, 0.2)) for name in self._scales() if name]
+
+    def load(self, fetch, runtime) -> None:
+        super().load(fetch, runtime)
+        self.scales = [fetch(name) if name else torch.ones((self.width,), dtype=torch.float32, device=runtime.device)
+                       for name in self._scales()]
+
+    def forward(self, stream: ResidualStream, step, cache: LayerCache | None) -> None:
+        x = stream.rows(self.runtime.dtype)
+        y = _float32_product(self.mixer.forward(x, step, cache))
+        h = stream.settle()
+        with stage("sum, norm"):
+            x = self.mixer_norm.join_normed(h, y, self.scales[0], self.alpha)
+        if self.feed_forward is not None:
+            y = _float32_product(self.feed_forward.forward(x, step))
+            with stage("sum, norm"):
+                x = self.ffn_norm.join_normed(h, y, self.scales[1], self.alpha)
+        stream.rewritten(x if x.dtype != torch.float32 else None)
+
+
 class HyperConnectionBlock(Block):
     """A pre-norm layer around ``streams`` residual streams instead of one.  For sublayer q (the mixer, then the
     feed-forward) with its three tensors ``in`` [S], ``mix`` [S, S] (from, to) and ``out`` [S]:

@@ -147,9 +147,9 @@ class PolyNormFF(FeedForward):
 
 
 class ActivatedFF(FeedForward):
-    """y = down(act(up(x) + b_up)) + b_down without a gate, act an element-wise unit with stored numbers of its own.
+    """y = down(act(up(x) + b_up)) + b_down without a gate, act an element-wise unit, perhaps with stored numbers of its own.
 
-    ``activation`` "xielu": with the two stored numbers (p, q) of the ``act`` tensor,
+    ``activation`` "squared_relu": act(z) = max(z, 0)^2, no stored numbers.  "xielu": with the two stored numbers (p, q) of the ``act`` tensor,
 
         act(z) = softplus(p) z^2 + z / 2                          for z > 0,
                  (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2     for z <= 0.
@@ -159,7 +159,7 @@ class ActivatedFF(FeedForward):
     graph_safe = True
 
     ROLES = {"up": "up", "down": "down", "act": "act"}
-    ACTIVATIONS = {"xielu": 2}          # name -> how many numbers it stores
+    ACTIVATIONS = {"xielu": 2, "squared_relu": 0}          # name -> how many numbers it stores
 
     def __init__(self, prefix: str, hidden_size: int, intermediate_size: int, activation: str = "xielu", bias: bool = True,
                  names: dict[str, str] | None = None, suffix: str = "weight", bias_suffix: str = "bias") -> None:
@@ -182,8 +182,9 @@ class ActivatedFF(FeedForward):
 
     def weight_specs(self) -> list[WeightSpec]:
         h, i = self.hidden_size, self.intermediate_size
-        specs = [WeightSpec(self._tensor("up"), (i, h), MATRIX), WeightSpec(self._tensor("down"), (h, i), MATRIX),
-                 WeightSpec(self.name(self.names["act"]), (self.ACTIVATIONS[self.activation],), VECTOR, Init(0.3, 0.3))]
+        specs = [WeightSpec(self._tensor("up"), (i, h), MATRIX), WeightSpec(self._tensor("down"), (h, i), MATRIX)]
+        if self.ACTIVATIONS[self.activation]:
+            specs.append(WeightSpec(self.name(self.names["act"]), (self.ACTIVATIONS[self.activation],), VECTOR, Init(0.3, 0.3)))
         if self.bias:
             specs += [WeightSpec(self._bias("up"), (i,), VECTOR), WeightSpec(self._bias("down"), (h,), VECTOR)]
         return specs
@@ -192,7 +193,7 @@ class ActivatedFF(FeedForward):
         super().load(fetch, runtime)
         self.up = Projection(fetch(self._tensor("up")), fetch(self._bias("up")) if self.bias else None, label="up")
         self.down = Projection(fetch(self._tensor("down")), fetch(self._bias("down")) if self.bias else None, label="down")
-        self.numbers = fetch(self.name(self.names["act"]))
+        self.numbers = fetch(self.name(self.names["act"])) if self.ACTIVATIONS[self.activation] else None
 
     def flops(self, tokens: int, attended: int) -> float:
         return self.up.flops(tokens) + self.down.flops(tokens)
@@ -203,5 +204,8 @@ class ActivatedFF(FeedForward):
         with stage(self.up.label):
             z = linear_kernels.linear(x, self.up.weight, self.up.bias, torch.float32)
         with stage("activation"):
-            a = ops.xielu(z, self.numbers, self.runtime.dtype)
+            if self.activation == "squared_relu":
+                a = ops.squared_relu(z, self.runtime.dtype)
+            else:
+                a = ops.xielu(z, self.numbers, self.runtime.dtype)
         return self.down.deferred(a)

@@ -3,8 +3,9 @@
 Router: ``z = W_r x`` in float32 and scores ``s = softmax(z)`` over all experts, or ``s = sigmoid(z)`` expert by expert
 (``scores``).  The experts come in ``groups`` equal runs of neighbours; a run scores as its best expert, and only
 experts of the ``keep`` best runs can be chosen.  Of those the ``top`` with the largest s are taken, weighted by s over
-the sum of the chosen scores (+ 1e-20) or by s as it is (``normalize``).  With a ``correction`` tensor, one number an
-expert, the choice looks at s + correction and the weights at s alone.  A gated expert is
+the sum of the chosen scores (+ 1e-20) or by s as it is (``normalize``; of a softmax over all experts that is the softmax
+over the chosen ones).  With a ``correction`` tensor, one number an expert, the choice looks at s + correction and the
+weights at s alone; with ``router_bias`` a stored number an expert is part of z.  A gated expert is
 
     g = min(W_gate x, limit);  u = clamp(W_up x, -limit, limit);  y = W_down (g sigmoid(alpha g) (u + shift))
 
@@ -12,7 +13,8 @@ without biases (no ``limit``, alpha 1 and shift 0: the plain ``silu(W_gate x) * 
 "squared_relu") is ``y = W_down relu(W_up x)^2``.  The output is the weighted
 sum of the chosen experts' outputs or, with ``weight_on="input"``, the sum of the experts applied to ``w x`` (the
 weight then scales the float32 sums of gate and up before the unit, which is not the same thing since the unit is not
-linear); plus the shared expert's (the same form with sizes and a limit of its own).  The (token, expert) pairs are sorted by expert on the device, so that an
+linear); plus the shared expert's (the same form with sizes and a limit of its own), with ``shared_gate`` times sigmoid(w
+x), one number a token.  The (token, expert) pairs are sorted by expert on the device, so that an
 expert's rows are one block of the products' input; nothing of it is read by the host.
 """
 
@@ -41,7 +43,7 @@ class RoutedExperts(FeedForward):
     graph_safe = True
 
     ROLES = {"router": "router", "expert": "e", "shared": "shared", "gate": "gate", "up": "up", "down": "down",
-             "correction": "correction"}
+             "correction": "correction", "bias": "router.b", "shared_gate": "sg"}
 
     UNITS = ("clamped_glu", "squared_relu")
     SCORES = ("softmax", "sigmoid")
@@ -51,9 +53,9 @@ class RoutedExperts(FeedForward):
                  groups: int = 1, keep_groups: int = 1, shared_size: int | None = None, shared_limit: float | None = None,
                  alpha: float = 1.702, shift: float = 1.0, names: dict[str, str] | None = None, suffix: str = "weight",
                  scores: str = "softmax", normalize: bool = True, weight_on: str = "output", unit: str = "clamped_glu",
-                 correction: bool = False) -> None:
+                 correction: bool = False, router_bias: bool = False, shared_gate: bool = False) -> None:
         """``names``: ``router``, the experts' stem (``e`` gives ``e0``, ``e1``, ...), ``shared``, the three matrices
-        of an expert (two without a gate) and ``correction``; ``suffix`` follows a matrix's name (empty: nothing)."""
+        of an expert (two without a gate), ``correction``, ``bias`` and the shared expert's ``shared_gate``; ``suffix`` follows a matrix's name (empty: nothing)."""
         super().__init__(prefix)
         unknown = set(names or {}) - set(self.ROLES)
         if unknown:
@@ -73,6 +75,9 @@ class RoutedExperts(FeedForward):
         if unit not in self.UNITS:
             raise ValueError(f"{prefix}: an expert's unit is one of {self.UNITS}, got {unit!r}")
         self.gated, self.has_correction = unit == "clamped_glu", bool(correction)
+        self.has_bias, self.has_shared_gate = bool(router_bias), bool(shared_gate)
+        if self.has_shared_gate and not shared_size:
+            raise ValueError(f"{prefix}: a gate on the shared expert needs a shared expert")
         self.unit = ClampedGLU(limit, alpha, shift)
         self.shared_size = int(shared_size) if shared_size else None
         self.shared_unit = ClampedGLU(shared_limit if shared_limit is not None else limit, alpha, shift) if self.shared_size else None
@@ -93,6 +98,10 @@ class RoutedExperts(FeedForward):
         specs = [WeightSpec(self._matrix(self.names["router"]), (self.num_experts, h), VECTOR)]
         if self.has_correction:
             specs.append(WeightSpec(self.name(self.names["correction"]), (self.num_experts,), VECTOR, Init(0.0, 0.02)))
+        if self.has_bias:
+            specs.append(WeightSpec(self.name(self.names["bias"]), (self.num_experts,), VECTOR, Init(0.0, 0.1)))
+        if self.has_shared_gate:
+            specs.append(WeightSpec(self._matrix(self.names["shared"], self.names["shared_gate"]), (1, h), VECTOR))
         feeds = [(self._expert(e), self.expert_size) for e in range(self.num_experts)]
         if self.shared_size:
             feeds.append((self.names["shared"], self.shared_size))
@@ -104,6 +113,10 @@ class RoutedExperts(FeedForward):
     def load(self, fetch: Fetch, runtime: Runtime) -> None:
         super().load(fetch, runtime)
         self.router = fetch(self._matrix(self.names["router"]))            # float32: the router is computed in 32-bit
+        if self.has_shared_gate:                                          # one row more of the router's product
+            gate = fetch(self._matrix(self.names["shared"], self.names["shared_gate"]))
+            self.router = torch.cat([self.router, gate], dim=0).contiguous()
+        self.router_bias = fetch(self.name(self.names["bias"])) if self.has_bias else None
         self.correction = fetch(self.name(self.names["correction"])) if self.has_correction else None
         up, down = [], []
         for e in range(self.num_experts):
@@ -128,8 +141,9 @@ class RoutedExperts(FeedForward):
         if hasattr(x, "materialize"):
             x = x.materialize()
         with stage("router"):
+            gate = (torch.empty((x.shape[0],), dtype=torch.float32, device=x.device) if self.has_shared_gate else None)
             chosen, weight = ops.moe_route(x, self.router, self.top, self.groups, self.keep_groups, self.scores,
-                                           self.normalize, self.correction)
+                                           self.normalize, self.correction, self.router_bias, gate)
             # bfloat16: the products run on the matrix cores, in tiles sized by the rows an expert gets in this step
             mfma = ops.moe_mfma_supported(x, self.up, self.down)
             rows = ops.moe_tile_rows(chosen.numel(), self.num_experts, mfma)
@@ -146,7 +160,7 @@ class RoutedExperts(FeedForward):
                                  tile_rows=rows, mfma=mfma)
         shared = self._shared(x) if self.shared_size else None
         with stage("experts' sum"):
-            return ops.moe_combine(pairs, self.top, shared)
+            return ops.moe_combine(pairs, self.top, shared, gate)
 
     def _shared(self, x: torch.Tensor) -> torch.Tensor:
         if not self.gated:

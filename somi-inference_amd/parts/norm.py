@@ -46,6 +46,10 @@ class RMSNorm(Norm):
         y = y if y.dtype == torch.float32 else y.to(torch.float32)
         return ops.normed_add(h, y, self.weight, self.eps, 1.0, copy_dtype)
 
+    def join_normed(self, h: torch.Tensor, y: torch.Tensor, scale: torch.Tensor, alpha: float) -> torch.Tensor:
+        copy = ops.join_norm(h, y, scale, alpha, self.weight, self.eps, self.runtime.dtype == torch.bfloat16)
+        return h if copy is None else copy
+
 
 class DynamicTanh(Norm):
     """y = tanh(alpha * x) * w + b: a norm that computes no mean and no variance.  ``alpha`` is one stored number,

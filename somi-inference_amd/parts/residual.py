@@ -26,6 +26,7 @@ class ResidualStream:
         assert h.dtype == torch.float32 and h.dim() == 2
         self.h = h
         self._pending: torch.Tensor | DeferredProduct | None = None
+        self._rounded: torch.Tensor | None = None   # h in the compute dtype, if whoever wrote h last left it
         self.lanes: torch.Tensor | None = None      # [S, N, H] float32 once a layer keeps several streams side by side
 
     def fan_out(self, count: int) -> torch.Tensor:
@@ -43,10 +44,25 @@ class ResidualStream:
         if self.lanes is not None:
             raise RuntimeError("the stream runs as several streams side by side; this layer's arrangement knows one")
 
+    def rows(self, dtype: torch.dtype) -> torch.Tensor:
+        """The stream itself in ``dtype``, for sublayers that read it without a norm (float32: the rows, not a copy)."""
+        self._single()
+        h = self.settle()
+        if dtype == torch.float32:
+            return h
+        if self._rounded is None or self._rounded.dtype != dtype:
+            self._rounded = h.to(dtype)
+        return self._rounded
+
+    def rewritten(self, rounded: torch.Tensor | None = None) -> None:
+        """``h`` has been written in place; ``rounded``: the new rows in the compute dtype, if there are any."""
+        self._rounded = rounded
+
     def add(self, delta: "torch.Tensor | DeferredProduct") -> None:
         """Queue ``h += delta``."""
         self._single()
         self.settle()
+        self._rounded = None
         self._pending = delta
 
     def normed(self, norm: Norm, lazy: bool = False) -> "torch.Tensor | NormedRows":

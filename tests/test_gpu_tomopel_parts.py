@@ -243,7 +243,7 @@ def test_sizes_without_a_matrix_core_kernel_for_the_bias_are_refused_by_it():
     kc, vc, table = paged(20, 1, 144, 8, gen)
     q = torch.randn(20, 144, generator=gen).to(torch.bfloat16).to(DEV)
     bias = torch.zeros(1, 5, device=DEV)
-    assert not attention_kernels.bias_supported(kc, table)
+    assert not attention_kernels.forms_supported(kc, table)
     entry, positions = torch.zeros(20, dtype=torch.int32, device=DEV), torch.arange(20, dtype=torch.int32, device=DEV)
     with pytest.raises(ops.KernelError, match="distance bias"):
         ops.attention_decode(q, 144, kc, vc, table, entry, positions, 1, 0, 0.1, 64, 1, torch.empty_like(q), bias=bias)
