@@ -36,7 +36,7 @@ def pusazen_plan(config: PusazenConfig) -> ModelPlan:
                                                      "value_dim": m.vdim, "decay": m.decay, "eps": config.norm_eps, "suffix": ""})
         else:
             position = (PartSpec("none", {}) if m.rot_base is None else
-                        PartSpec("rotary", {"head_dim": m.dim, "theta": m.rot_base, "rotary_dim": m.rot_dims}))
+                        PartSpec("rotary", {"head_dim": m.dim, "theta": m.rot_base, "rotary_dim": m.rot_dims, "double": True}))
             mixer = PartSpec("gqa_attention", {
                 "hidden_size": config.width, "num_heads": m.heads, "num_kv_heads": m.kv_heads, "head_dim": m.dim,
                 "value_dim": m.vdim, "position": position, "qkv_bias": False, "scale": m.scale, "qk_norm": "projection",

@@ -54,10 +54,12 @@ class RotaryPosition(PositionEncoding):
     PAIRINGS = ("half", "neighbours")
 
     def __init__(self, prefix: str, head_dim: int, theta: float, rotary_dim: int | None = None,
-                 pairing: str = "half", scaling: dict | None = None) -> None:
+                 pairing: str = "half", scaling: dict | None = None, double: bool = False) -> None:
+        """``double``: the frequencies are computed in double precision and rounded once, also where the reference's own
+        arithmetic (float32 powers) would do."""
         super().__init__(prefix)
         self.head_dim = int(head_dim)
-        self.theta = float(theta)
+        self.theta, self.double = float(theta), bool(double)
         self.rotary_dim = int(rotary_dim if rotary_dim is not None else head_dim)
         if self.rotary_dim % 2 or not 0 < self.rotary_dim <= self.head_dim:
             raise ValueError(f"rotary_dim {self.rotary_dim} must be even and within head_dim {self.head_dim}")
@@ -90,7 +92,7 @@ class RotaryPosition(PositionEncoding):
 
     def load(self, fetch: Fetch, runtime: Runtime) -> None:
         super().load(fetch, runtime)
-        if self.scaling is None and self.ramp is None and self.pairing == "half":
+        if self.scaling is None and self.ramp is None and self.pairing == "half" and not self.double:
             # the reference's own arithmetic (float32 powers), bit for bit
             exponents = torch.arange(0, self.rotary_dim, 2, dtype=torch.float32) / self.rotary_dim
             self.inv_freq = (1.0 / (self.theta ** exponents)).to(runtime.device)

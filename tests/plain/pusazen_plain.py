@@ -167,23 +167,27 @@ def experts(x: torch.Tensor, weights: dict, prefix: str, mlp: dict, margins: lis
 
 
 # ------------------------------------------------------------------------------------- the model
-def forward(config: dict, weights: dict, tokens: list[int], dtype=torch.float64,
-            margins: list | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+def forward(config: dict, weights: dict, tokens: list[int], dtype=torch.float64, margins: list | None = None,
+            read_as: torch.dtype | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """Logits [T, vocab] and the stream after every layer [layers, T, width].  ``margins`` collects, per routed layer,
-    how far each token's choice of experts was from another one."""
+    how far each token's choice of experts was from another one.  ``read_as``: what the sublayers read is rounded to this
+    type (how much rounding alone moves a row)."""
+    def read(x: torch.Tensor) -> torch.Tensor:
+        return x if read_as is None else x.to(read_as).to(dtype)
+
     w = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in weights.items()}
     eps, alpha = float(config["norm"]["eps"]), float(config["postln_alpha"])
     x = w["embed"][torch.tensor(tokens)]
     after = []
     for n, layer in enumerate(config["layers"]):
         p, mlp = f"l{n}.", layer.get("mlp")
-        y = MIXERS[layer["type"]](x, w, p + "mix.", layer["mixer"], eps)
+        y = MIXERS[layer["type"]](read(x), w, p + "mix.", layer["mixer"], eps)
         x = norm_after(x, y, w[p + "ls1"], alpha, w[p + "norm1"], eps)
         if mlp:
-            y = dense(x, w, p + "mlp.") if mlp["kind"] == "dense" else experts(x, w, p + "mlp.", mlp, margins)
+            y = dense(read(x), w, p + "mlp.") if mlp["kind"] == "dense" else experts(read(x), w, p + "mlp.", mlp, margins)
             x = norm_after(x, y, w[p + "ls2"], alpha, w[p + "norm2"], eps)
         after.append(x)
-    return (rms(x, eps) * w["final.norm"]) @ w["head"].T * float(config["logit_scale"]), torch.stack(after)
+    return read(rms(x, eps) * w["final.norm"]) @ w["head"].T * float(config["logit_scale"]), torch.stack(after)
 
 
 def load_folder(folder: str, dtype=torch.float32) -> tuple[dict, dict]:

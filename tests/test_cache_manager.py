@@ -262,3 +262,28 @@ def test_a_group_stores_what_its_spec_lists_in_pages_of_its_own_size():
 def _reserved(m, request_id, count):
     m.reserve(request_id, count)
     return m
+
+
+def test_chunked_group_gives_back_the_pages_before_a_chunk():
+    """Chunks of 10 over pages of 4: page p is done once the next token's chunk starts at or beyond its end."""
+    needs = [PagedKVSpec(1, 8), PagedKVSpec(1, 8, chunk=10), PagedKVSpec(1, 8, chunk=10, window=6), PagedKVSpec(1, 8, chunk=10)]
+    m = CacheManager(needs, block_size=4, num_blocks=12, max_requests=2, dtype=torch.float32, device="cpu", allocate_tensors=False)
+    assert [(g.window, g.chunk, g.runs) for g in m.groups] == [(None, None, [0]), (None, 10, [1, 3]), (6, 10, [2])]
+    m.register("a")
+    for tokens, chunked, both in ((9, [0, 1, 2], [1, 2]), (10, [2], [2]), (12, [2], [2]), (19, [2, 3, 4], [3, 4]), (20, [], []),
+                                  (21, [5], [5]), (33, [7, 8], [7, 8])):
+        new = tokens - m.num_tokens("a")
+        m.reserve("a", new)
+        m.commit("a", new)
+        held = [[i for i, page in enumerate(m.page_list(g, "a")) if page != -1] for g in range(3)]
+        assert held == [list(range((tokens + 3) // 4)), chunked, both], tokens
+        m.check_invariants()
+    m.free("a")
+    m.check_invariants()
+    assert m.free_pages() == [12, 12, 12]
+
+
+def test_a_chunk_comes_without_kept_first_tokens():
+    for bad in (dict(chunk=0), dict(chunk=4, keep_first=2)):
+        with pytest.raises(ValueError):
+            PagedSpec((PageTensor("latent", (PAGE, 4)),), **bad)
