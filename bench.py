@@ -285,6 +285,42 @@ def tomopel_closest_streams_config_dict(sizes: str) -> dict:
             "layers": [layer] * TOMOPEL_LAYERS}
 
 
+# layer sizes of Pusazen models that resemble real ones: (width, mLSTM heads, their key and value sizes, lightning heads, their
+# key and value sizes, attention heads, key/value heads, head size, chunk, experts, experts a token, an expert's size, the
+# shared expert's size, the dense feed-forward's size, vocabulary).  Six layers: three mLSTM, two attention, one lightning; a
+# dense feed-forward in the first, routed experts in the others.  The states hold as many elements as the Mamba-2 states of the
+# Tomopel model of the same name.
+PUSAZEN_SIZES = {
+    "1b": (2048, 8, 128, 256, 16, 128, 128, 16, 4, 128, 8192, 32, 4, 512, 1024, 8192, 32000),
+    "7b": (4096, 16, 128, 256, 32, 128, 128, 32, 8, 128, 8192, 64, 6, 1024, 2048, 16384, 32000),
+}
+PUSAZEN_LAYERS = {"mlstm": 3, "attention": 2, "lightning": 1}
+
+
+def pusazen_config_dict(sizes: str) -> dict:
+    (width, m_heads, m_dim, m_vdim, l_heads, l_dim, l_vdim, heads, kv_heads, dim, chunk, experts, top, ff, shared, dense_ff,
+     vocab) = PUSAZEN_SIZES[sizes]
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff}, "shared": {"ff": shared}}
+    mixers = {"mlstm": {"heads": m_heads, "dim": m_dim, "vdim": m_vdim, "gate_cap": 15.0},
+              "lightning": {"heads": l_heads, "dim": l_dim, "vdim": l_vdim, "decay": [1.0 - 2.0 ** -(2 + h % 8) for h in range(l_heads)]},
+              "attention": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "softcap": 50.0,
+                            "rot": {"base": 10000.0, "dims": dim // 2}, "mask": {"size": chunk}}}
+    order = ("mlstm", "attention", "mlstm", "lightning", "mlstm", "attention")
+    return {"architecture": "Pusazen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "postln_alpha": 2.0, "logit_scale": 1.0,
+            "layers": [{"type": kind, "mixer": mixers[kind], "mlp": moe if index else {"kind": "dense", "ff": dense_ff}}
+                       for index, kind in enumerate(order)]}
+
+
+def pusazen_closest_dense_config_dict(sizes: str) -> dict:
+    """The closest model for the ungated dense feed-forward and for the norm behind a sublayer: a Metitar model of the same
+    width whose layers all have a dense feed-forward of the same size."""
+    (width, m_heads, m_dim, m_vdim, l_heads, l_dim, l_vdim, heads, kv_heads, dim, chunk, experts, top, ff, shared, dense_ff,
+     vocab) = PUSAZEN_SIZES[sizes]
+    layer = {"type": "hgrn2", "mixer": {"heads": l_heads, "dim": l_dim, "vdim": l_vdim}, "mlp": {"kind": "dense", "ff": dense_ff}}
+    return {"architecture": "Metitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": [layer] * 6}
+
+
 # keys of a config.json that name sizes, in the order they are reported under "config" (flat, at most 20 keys)
 SIZE_KEYS = ("hidden_size", "intermediate_size", "num_attention_heads", "num_key_value_heads", "head_dim",
              "vocab_size", "tie_word_embeddings")
@@ -334,6 +370,10 @@ def parse_args() -> argparse.Namespace:
                         "streams, attention with mixed heads, windowed attention over a shared latent) at these layer "
                         "sizes, beside a Metitar model of equal width, latent and feed-forwards and a Qwen2.5-style model "
                         "of equal width, heads and window, each with its stage times")
+    p.add_argument("--pusazen", default=None, choices=sorted(PUSAZEN_SIZES), metavar="SIZES",
+                   help="instead of the default workload: prefill and decode of a Pusazen model (mLSTM, lightning attention, "
+                        "chunked attention with capped scores and a sink, gated experts) at these layer sizes beside the "
+                        "closest models of the engine")
     p.add_argument("--tomopel", default=None, choices=sorted(TOMOPEL_SIZES), metavar="SIZES",
                    help="instead of the default workload: prefill and decode of a Tomopel model (attention with a distance "
                         "bias beside Mamba-2, minGRU, ungated experts, several residual streams) at these layer sizes, "
@@ -1063,6 +1103,101 @@ def run_tomopel(args) -> dict:
     return out
 
 
+def run_pusazen(args) -> dict:
+    """Prefill and decode of a Pusazen model beside the closest models the engine had (Tomopel: the recurrence, the attention
+    and what normed heads take; Rusolorn: gated experts; Metitar: an ungated dense feed-forward and a norm behind a sublayer),
+    with the stage times of all four and what the kernels reach of the machine."""
+    (width, m_heads, m_dim, m_vdim, l_heads, l_dim, l_vdim, heads, kv_heads, dim, chunk, experts, top, ff, shared, dense_ff,
+     vocab) = PUSAZEN_SIZES[args.pusazen]
+    (_, t_streams, t_heads, t_kv, t_dim, r_heads, r_vdim, r_state, *_) = TOMOPEL_SIZES[args.pusazen]
+    batches, context, tokens = (8, 64), args.context, args.prefill_tokens
+    out: dict = {}
+    for label, config_dict in (("pusazen", pusazen_config_dict(args.pusazen)), ("closest", tomopel_config_dict(args.pusazen)),
+                               ("closest_experts", tomopel_closest_config_dict(args.pusazen)),
+                               ("closest_dense", pusazen_closest_dense_config_dict(args.pusazen))):
+        bench = Workbench(config_dict, dtype=args.dtype, seed=args.seed, block_size=args.block_size,
+                          pool_tokens=Workbench.pool_tokens(batches, context, tokens), max_requests=max(batches))
+        block: dict = {"prefill": {str(n): bench.prefill_run(n) for n in sorted({512, tokens})}}
+        for batch in batches:
+            run = bench.decode_run(batch, max(POINT_MIN_STEPS, args.steps // 2), max(2, args.warmup // 2), context)
+            block[f"decode_b{batch}"] = {"tok_s": round(run["tok_s"], 1), "ms": round(run["ms"], 4),
+                                        "mean_ctx": round(run["mean_ctx"], 1)}
+        block["stages"] = bench.stage_run(tokens, batches[0], context)
+        print_stage_tables(block["stages"])
+        out[label] = block
+        bench.close()
+    bf16_peak = PEAK_FLOPS["bfloat16"]
+    count = PUSAZEN_LAYERS
+    layers, routed = sum(count.values()), sum(count.values()) - 1
+    theirs, t_mixed = TOMOPEL_LAYERS, TOMOPEL_PARALLEL
+
+    def stage_ms(label, run, *names):
+        return sum(out[label]["stages"][run].get(name, {}).get("ms", 0.0) for name in names)
+
+    def rate(flops, ms):
+        return {"ms": round(ms, 4), "tflops": round(flops / 1e9 / max(ms, 1e-9), 2),
+                "frac_of_peak": round(flops / 1e3 / max(ms, 1e-9) / bf16_peak * 1e6, 5)}
+
+    def stream(bytes_, ms):
+        return {"ms": round(ms, 4), "gbs": round(bytes_ / 1e6 / max(ms, 1e-9), 1)}
+    pairs = sum(p % chunk + 1 for p in range(tokens))
+    m_state, l_state, inner = m_heads * m_dim * (m_vdim + 1), l_heads * l_dim * l_vdim, r_heads * r_vdim
+    state = count["mlstm"] * m_state + count["lightning"] * l_state
+    mixed = count["mlstm"] * m_heads * m_vdim + count["lightning"] * l_heads * l_vdim
+    run = f"prefill_{tokens}"
+    out["prefill_kernels"] = {
+        "tokens": tokens,
+        "pusazen_attention": rate(count["attention"] * 4.0 * heads * dim * pairs, stage_ms("pusazen", run, "attention")),
+        "closest_attention": rate(t_mixed * 4.0 * t_heads * t_dim * tokens * (tokens + 1) / 2, stage_ms("closest", run, "attention")),
+        # per token and element of the state: its update and its product with q (or C)
+        "pusazen_recurrence": rate(4.0 * state * tokens, stage_ms("pusazen", run, "recurrence")),
+        "closest_recurrence": rate(t_mixed * 4.0 * inner * r_state * tokens, stage_ms("closest", run, "recurrence")),
+        "pusazen_gates": {"ms": round(stage_ms("pusazen", run, "gates"), 4)},
+        # q, k and v read and written in float32; x, B and C through a convolution
+        "pusazen_input_activation": stream(count["lightning"] * tokens * l_heads * (2 * l_dim + l_vdim) * 8.0, stage_ms("pusazen", run, "input activation")),
+        "closest_convolution": stream(t_mixed * tokens * (inner + 2 * r_state) * 8.0, stage_ms("closest", run, "convolution")),
+        # y and the gate read in float32, the normed rows written
+        "pusazen_norm_gate": stream(tokens * mixed * 10.0, stage_ms("pusazen", run, "norm, gate")),
+        "closest_gate_norm": stream(t_mixed * tokens * inner * 10.0, stage_ms("closest", run, "gate, norm")),
+        # the q/k/v sums read in float32, q, k and v written
+        "pusazen_qk_norm": stream(count["attention"] * tokens * (heads + 2 * kv_heads) * dim * 6.0,
+                                  stage_ms("pusazen", run, "q/k norm, position encoding, k/v into pages")),
+        "closest_head_norms": stream(t_mixed * tokens * (t_heads + 2 * t_kv) * t_dim * 6.0, stage_ms("closest", run, "head norms, k/v into pages")),
+        "pusazen_experts": rate(routed * 6.0 * tokens * top * ff * width, stage_ms("pusazen", run, "experts gate_up", "experts down")),
+        "closest_experts": rate(theirs * 6.0 * tokens * top * ff * width, stage_ms("closest_experts", run, "experts gate_up", "experts down")),
+        "pusazen_shared": rate(routed * 6.0 * tokens * shared * width, stage_ms("pusazen", run, "shared gate_up", "shared activation", "shared down")),
+        "closest_shared": rate(theirs * 6.0 * tokens * shared * width, stage_ms("closest_experts", run, "shared gate_up", "shared activation", "shared down")),
+        "pusazen_router": {"ms_a_layer": round(stage_ms("pusazen", run, "router") / routed, 4)},
+        "closest_router": {"ms_a_layer": round(stage_ms("closest_experts", run, "router") / theirs, 4)},
+        "pusazen_dense": rate(4.0 * tokens * dense_ff * width, stage_ms("pusazen", run, "up", "down", "activation")),
+        "closest_dense": rate(6 * 4.0 * tokens * dense_ff * width, stage_ms("closest_dense", run, "up", "down", "activation")),
+        "pusazen_mixer_products": rate(2.0 * tokens * width * (
+            count["mlstm"] * m_heads * (2 * m_dim + 3 * m_vdim + 2) + count["lightning"] * l_heads * (2 * l_dim + 3 * l_vdim)
+            + count["attention"] * (2 * heads + 2 * kv_heads) * dim), stage_ms("pusazen", run, "q/k/v/g/gates", "q/k/v/g", "q/k/v", "o")),
+        "closest_mixer_products": rate(theirs * 2.0 * tokens * width * 4 * l_heads * l_dim, stage_ms("closest_dense", run, "q/f/v", "o")),
+        # the stream read and written in float32, the sublayer's rows read, the new rows written once more in 16 bits
+        "pusazen_sum_norm": stream(2 * layers * tokens * width * (8.0 + 4 + 2), stage_ms("pusazen", run, "sum, norm")),
+        "closest_output_norm": stream(12 * tokens * width * (8.0 + 4 + 2), stage_ms("closest_dense", run, "output norm, residual add")),
+    }
+    run = f"decode_b{batches[0]}_eager"
+    used = min(experts, batches[0] * top)          # experts a step touches at most
+    seen = (context - 1) % chunk + 1
+    out["decode_kernels"] = {
+        "batch": batches[0], "context": context,
+        "pusazen_attention": stream(count["attention"] * batches[0] * seen * kv_heads * 2 * dim * 2.0, stage_ms("pusazen", run, "attention")),
+        "closest_attention": stream(t_mixed * batches[0] * context * t_kv * 2 * t_dim * 2.0, stage_ms("closest", run, "attention")),
+        "pusazen_recurrence": stream(batches[0] * state * 8.0, stage_ms("pusazen", run, "recurrence")),
+        "closest_recurrence": stream(t_mixed * batches[0] * inner * r_state * 8.0, stage_ms("closest", run, "recurrence")),
+        "pusazen_experts": stream(routed * used * 3.0 * ff * width * 2.0, stage_ms("pusazen", run, "experts gate_up", "experts down")),
+        "closest_experts": stream(theirs * used * 3.0 * ff * width * 2.0, stage_ms("closest_experts", run, "experts gate_up", "experts down")),
+        "pusazen_dense": stream(2.0 * dense_ff * width * 2.0, stage_ms("pusazen", run, "up", "down", "activation")),
+        "closest_dense": stream(6 * 2.0 * dense_ff * width * 2.0, stage_ms("closest_dense", run, "up", "down", "activation")),
+        "pusazen_sum_norm": {"ms_a_layer": round(stage_ms("pusazen", run, "sum, norm") / layers, 4)},
+        "closest_output_norm": {"ms_a_layer": round(stage_ms("closest_dense", run, "output norm, residual add") / 6, 4)},
+    }
+    return out
+
+
 def main() -> int:
     args = parse_args()
     world = int(os.environ.get("WORLD_SIZE", "1"))
@@ -1077,6 +1212,16 @@ def main() -> int:
                 "data": "synthetic: seeded random weights, seeded uniform token ids", "sizes": args.kamedra}
         line.update(run_kamedra(args))
         line["value"] = line["kamedra"][f"decode_b8"]["tok_s"]
+        line["seconds_total"] = round(time.perf_counter() - started, 1)
+        print(json.dumps(line))
+        return 0
+
+    if args.pusazen:
+        line = {"metric": f"Pusazen at {args.pusazen} layer sizes beside the closest Tomopel, Rusolorn and Metitar models: prefill and decode",
+                "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                "data": "synthetic: seeded random weights, seeded uniform token ids", "sizes": args.pusazen}
+        line.update(run_pusazen(args))
+        line["value"] = line["pusazen"]["decode_b8"]["tok_s"]
         line["seconds_total"] = round(time.perf_counter() - started, 1)
         print(json.dumps(line))
         return 0

@@ -409,9 +409,7 @@ attention_decode_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const 
             }
             if (SHAPED) {
 #pragma unroll
-                for (int half = 0; half < 2; ++half)
-#pragma unroll
-                    for (int i = 0; i < 4; ++i) s[half][i] = cap(s[half][i]);
+                for (int half = 0; half < 2; ++half) cap.apply<4>(s[half]);
             }
             // s[half][i] = S[key j0 + 16 half + 4 g + i][head r], still unscaled; keys outside the split are
             // masked (only the first and last step of a split can hold any)

@@ -461,9 +461,7 @@ attention_prefill_lds_kernel(const bf16* __restrict__ q, int64_t q_stride, const
 #pragma unroll
                 for (int qb = 0; qb < QB; ++qb)
 #pragma unroll
-                    for (int half = 0; half < 2; ++half)
-#pragma unroll
-                        for (int i = 0; i < 4; ++i) s[qb][half][i] = cap(s[qb][half][i]);
+                    for (int half = 0; half < 2; ++half) cap.apply<4>(s[qb][half]);
             }
             // scores stay unscaled; keys a query must not see are masked, which only steps that reach past the
             // wavefront's first query (or a window's or a chunk's lower edge) can hold

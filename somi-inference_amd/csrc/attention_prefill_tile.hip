@@ -268,8 +268,7 @@ prefill_tile_kernel(const bf16* __restrict__ q, int64_t q_stride, const bf16* __
             }
             if (SHAPED) {
                 const float point = m_run == -INFINITY ? 0.f : m_run;
-#pragma unroll
-                for (int r = 0; r < 16; ++r) sc[r] = cap(sc[r]) - point;
+                cap.apply<16>(sc, point);
             }
             if (j0 + 31 > w_first) {
                 const int lim = p_rel - j0;

@@ -26,8 +26,8 @@ __device__ __forceinline__ int score_first_key(int p, int window, int chunk) {
     return start > lo ? start : lo;
 }
 
-// A raw product in base-2 units, capped: L = c log2(e) tanh(x / c) for the scaled score x = raw * unit / log2(e), where
-// `unit` turns a raw product into base-2 units of an uncapped score.  tanh(y) = 1 - 2 / (exp(2 y) + 1), which is -1 and 1 at
+// A raw product in base-2 units, capped, less `point`: c log2(e) tanh(x / c) - point for the scaled score x = raw * unit /
+// log2(e), where `unit` turns a raw product into base-2 units of an uncapped score.  tanh(y) = 1 - 2 / (exp(2 y) + 1), which is -1 and 1 at
 // both ends without a clamp.
 struct ScoreCap {
     float top, twice, rate;  // c log2(e), twice that, and 2 unit / c: exp(2 x / c) = exp2(raw * rate)
@@ -38,8 +38,15 @@ struct ScoreCap {
         twice = 2.f * top;
         rate = on ? 2.f * unit_ / softcap : 0.f;
     }
-    __device__ __forceinline__ float operator()(float raw) const {
-        if (!on) return raw * unit;
-        return fmaf(-twice, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(raw * rate) + 1.0f), top);
+    // N products at once, so that the question whether there is a cap is asked once.
+    template <int N, typename V> __device__ __forceinline__ void apply(V& raw, float point = 0.f) const {
+        if (on) {
+            const float high = top - point;
+#pragma unroll
+            for (int i = 0; i < N; ++i) raw[i] = fmaf(-twice, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(raw[i] * rate) + 1.0f), high);
+        } else {
+#pragma unroll
+            for (int i = 0; i < N; ++i) raw[i] = fmaf(raw[i], unit, -point);
+        }
     }
 };

@@ -1107,11 +1107,11 @@ def qk_norm_store(rows: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tenso
 def qk_norm_rope_store(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, q_weight: torch.Tensor,
                        k_weight: torch.Tensor, eps: float, inv_freq: torch.Tensor | None, rotary_dim: int, heads: int,
                        kv_heads: int, dim: int, vdim: int, k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
-    """From rows [q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim)]: q and k RMS-normed over their whole
+    """From float32 rows [q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim)]: q and k RMS-normed over their whole
     projections, the first ``rotary_dim`` channels of their heads turned (channel j with j + rotary_dim / 2, by position *
     inv_freq[j]); k and v into the tokens' slots of ``k_cache`` [pages, kv_heads, page, padded] and ``v_cache`` [pages,
     kv_heads, padded, page] -> q [N, heads * padded] in the caches' dtype.  Channels past dim and vdim are zeros."""
-    _need(rows, "projected rows")
+    _need(rows, "projected rows", torch.float32)
     n = rows.shape[0]
     if rows.shape[1] < (heads + kv_heads) * dim + kv_heads * vdim:
         raise KernelError(f"qk_norm_rope_store: rows of {rows.shape[1]} values do not hold the projections")
@@ -1127,8 +1127,8 @@ def qk_norm_rope_store(rows: torch.Tensor, positions: torch.Tensor, slots: torch
     if inv_freq is not None:
         _need(inv_freq, "inv_freq", torch.float32, (rotary_dim // 2,))
     q = torch.empty((n, heads * padded), dtype=k_cache.dtype, device=rows.device)
-    _check(library().somi_qk_norm_rope_store(_ptr(rows), dtype_code(rows.dtype), ctypes.c_int64(rows.shape[1]), _ptr(positions),
-                                             _ptr(slots), _ptr(q_weight), _ptr(k_weight), ctypes.c_float(eps), _ptr(inv_freq),
+    _check(library().somi_qk_norm_rope_store(_ptr(rows), ctypes.c_int64(rows.shape[1]), _ptr(positions), _ptr(slots),
+                                              _ptr(q_weight), _ptr(k_weight), ctypes.c_float(eps), _ptr(inv_freq),
                                              int(rotary_dim), n, int(heads), int(kv_heads), int(dim), int(vdim), padded, _ptr(q),
                                              _ptr(k_cache), _ptr(v_cache), page, dtype_code(k_cache.dtype), _stream()))
     return q

@@ -85,7 +85,7 @@ class LightningAttention(RowsMixer):
         if cache is None or cache.state is None:
             raise ValueError(f"{self.prefix}: the recurrence needs a state slot per request")
         q, k, v, g = torch.split(rows, self.splits, dim=1)
-        with stage("activation"):
+        with stage("input activation"):
             ops.silu_columns_(rows[:, :sum(self.splits[:3])])
         with stage("recurrence"):
             y, _ = ops.ssd_memory(q, k, v, step, cache.state, keep=self.decays)

@@ -22,10 +22,12 @@ from __future__ import annotations
 
 import torch
 
+from ..kernels import linear as linear_kernels
 from ..kernels import ops
 from ..kernels.stages import stage
 from ..weights.spec import MATRIX, VECTOR, Init, WeightSpec
 from .base import FeedForward, Fetch, Runtime
+from .feed_forward import SwiGLU
 from .linear import Projection
 
 
@@ -37,6 +39,7 @@ class ClampedGLU:
         self.alpha, self.shift = float(alpha), float(shift)
         if not self.limit > 0.0:
             raise ValueError(f"a clamp limit must be > 0, got {limit}")
+        self.plain = self.limit == float("inf") and self.alpha == 1.0 and self.shift == 0.0      # silu(g) u
 
 
 class RoutedExperts(FeedForward):
@@ -124,8 +127,14 @@ class RoutedExperts(FeedForward):
             down.append(fetch(self._matrix(self._expert(e), self.names["down"])))
         self.up = torch.stack(up).contiguous()                            # [experts, (2) F, H], gate rows first
         self.down = torch.stack(down).contiguous()                        # [experts, H, F]
-        self.shared_up = self.shared_down = None
-        if self.shared_size:
+        self.shared_up = self.shared_down = self.shared_glu = None
+        if self.shared_size and self.gated and self.shared_unit.plain:
+            # the plain gated unit: the product that ends in it
+            self.shared_glu = SwiGLU(self.name(self.names["shared"]), self.hidden_size, self.shared_size,
+                                     {role: self.names[role] for role in ("gate", "up", "down")}, suffix=self.suffix)
+            self.shared_glu.load(fetch, runtime)
+            self.shared_glu.gate_up.label, self.shared_glu.down.label = "shared gate_up", "shared down"
+        elif self.shared_size:
             s = self.names["shared"]
             self.shared_up = Projection.stacked([fetch(self._matrix(s, self.names[role])) for role in self._ups()],
                                                 label="shared gate_up" if self.gated else "shared up")
@@ -163,12 +172,18 @@ class RoutedExperts(FeedForward):
             return ops.moe_combine(pairs, self.top, shared, gate)
 
     def _shared(self, x: torch.Tensor) -> torch.Tensor:
+        if self.shared_glu is not None:
+            y = self.shared_glu.forward(x)
+            if hasattr(y, "projection"):
+                with stage(y.projection.label):
+                    return linear_kernels.linear(y.x, y.projection.weight, None, torch.float32)
+            return y
         if not self.gated:
             up = self.shared_up(x, torch.float32)
-            with stage("activation"):
+            with stage("shared activation"):
                 act = ops.squared_relu(up, self.runtime.dtype)
             return self.shared_down(act, torch.float32)
         gate_up = self.shared_up(x)
-        with stage("activation"):
+        with stage("shared activation"):
             gated = ops.clamped_glu(gate_up, self.shared_unit.limit, self.shared_unit.alpha, self.shared_unit.shift)
         return self.shared_down(gated)
