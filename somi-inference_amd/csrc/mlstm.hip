@@ -12,20 +12,18 @@
 // What leaves is made from the maxima as they were computed, so that the scan's rounding cancels between neighbours.
 #include "common.h"
 
-#define MLSTM_THREADS 256
-#define MLSTM_PER 4                  // neighbouring tokens of a thread
-
-// SOLO: every entry is a single token, 256 heads of one entry to a workgroup.
-template <bool SOLO>
-__global__ void __launch_bounds__(MLSTM_THREADS)
+// THREADS, PER: a workgroup's threads and the neighbouring tokens of each.  SOLO: entries of a few tokens, walked one by one
+// by a thread a head, THREADS heads of one entry to a workgroup.
+template <int THREADS, int PER, bool SOLO>
+__global__ void __launch_bounds__(THREADS)
 mlstm_gates_kernel(const float* __restrict__ ri, const float* __restrict__ rf, int64_t row_stride, const float* __restrict__ bi,
                    const float* __restrict__ bf, float cap, const int* __restrict__ entry_start,
                    const int* __restrict__ state_slots, float* __restrict__ top, int heads, float* __restrict__ keep,
                    float* __restrict__ write, float* __restrict__ floor_) {
-    constexpr int WAVES = MLSTM_THREADS / 64;
-    __shared__ float wave_f[WAVES], wave_g[WAVES], last[MLSTM_THREADS];
+    constexpr int WAVES = THREADS / 64;
+    __shared__ float wave_f[WAVES], wave_g[WAVES], last[THREADS];
     const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int h = SOLO ? blockIdx.y * MLSTM_THREADS + tid : blockIdx.y;
+    const int h = SOLO ? blockIdx.y * THREADS + tid : blockIdx.y;
     if (h >= heads) return;
     const int t0 = entry_start[e], t1 = entry_start[e + 1];
     float* kept = top + (int64_t)state_slots[e] * heads + h;
@@ -53,12 +51,12 @@ mlstm_gates_kernel(const float* __restrict__ ri, const float* __restrict__ rf, i
         *kept = m0;
         return;
     }
-    for (int base = t0; base < t1; base += MLSTM_THREADS * MLSTM_PER) {
-        float i[MLSTM_PER], f[MLSTM_PER];
+    for (int base = t0; base < t1; base += THREADS * PER) {
+        float i[PER], f[PER];
         float F = 0.f, G = -INFINITY;                        // this thread's tokens as one map
 #pragma unroll
-        for (int j = 0; j < MLSTM_PER; ++j) {
-            const int t = base + tid * MLSTM_PER + j;
+        for (int j = 0; j < PER; ++j) {
+            const int t = base + tid * PER + j;
             i[j] = -INFINITY;                                // a token past the entry's last: the map that changes nothing
             f[j] = 0.f;
             if (t < t1) gates(t, i[j], f[j]);
@@ -82,19 +80,19 @@ mlstm_gates_kernel(const float* __restrict__ ri, const float* __restrict__ rf, i
         for (int w = 0; w < wave; ++w) m = fmaxf(m + wave_f[w], wave_g[w]);
         const float pf = __shfl_up(F, 1, 64), pg = __shfl_up(G, 1, 64);
         if (lane > 0) m = fmaxf(m + pf, pg);
-        float ms[MLSTM_PER];
+        float ms[PER];
 #pragma unroll
-        for (int j = 0; j < MLSTM_PER; ++j) ms[j] = m = fmaxf(f[j] + m, i[j]);
+        for (int j = 0; j < PER; ++j) ms[j] = m = fmaxf(f[j] + m, i[j]);
         last[tid] = m;
         __syncthreads();
         float before = tid > 0 ? last[tid - 1] : m0;
 #pragma unroll
-        for (int j = 0; j < MLSTM_PER; ++j) {
-            const int t = base + tid * MLSTM_PER + j;
+        for (int j = 0; j < PER; ++j) {
+            const int t = base + tid * PER + j;
             if (t < t1) leave(t, i[j], f[j], before, ms[j]);
             before = ms[j];
         }
-        m0 = last[MLSTM_THREADS - 1];
+        m0 = last[THREADS - 1];
         __syncthreads();                                     // the reads, before the next tokens' maxima
     }
     if (tid == 0) *kept = m0;
@@ -108,12 +106,13 @@ extern "C" int somi_mlstm_gates(const float* ri, const float* rf, int64_t row_st
     SOMI_REQUIRE(n_entries >= 0 && heads > 0 && heads <= 65535 && row_stride >= heads, "mlstm_gates: bad sizes");
     SOMI_REQUIRE(cap > 0.f, "mlstm_gates: the gates' cap must be > 0, got %g", (double)cap);
     if (n_entries == 0) return 0;
-    if (max_entry_len <= 4)
-        hipLaunchKernelGGL(mlstm_gates_kernel<true>, dim3(n_entries, ceil_div(heads, MLSTM_THREADS)), dim3(MLSTM_THREADS), 0, stream, ri,
-                           rf, row_stride, bi, bf, cap, entry_start, state_slots, top, heads, keep, write, floor_);
-    else
-        hipLaunchKernelGGL(mlstm_gates_kernel<false>, dim3(n_entries, heads), dim3(MLSTM_THREADS), 0, stream, ri, rf, row_stride, bi, bf,
-                           cap, entry_start, state_slots, top, heads, keep, write, floor_);
+#define SOMI_MLSTM(THREADS, PER, SOLO, GRID_Y)                                                                                \
+    hipLaunchKernelGGL((mlstm_gates_kernel<THREADS, PER, SOLO>), dim3(n_entries, GRID_Y), dim3(THREADS), 0, stream, ri, rf,  \
+                       row_stride, bi, bf, cap, entry_start, state_slots, top, heads, keep, write, floor_)
+    if (max_entry_len <= 4) SOMI_MLSTM(256, 1, true, ceil_div(heads, 256));
+    else if (max_entry_len <= 512) SOMI_MLSTM(256, 2, false, heads);
+    else SOMI_MLSTM(1024, 2, false, heads);
+#undef SOMI_MLSTM
     SOMI_LAUNCH_CHECK("mlstm_gates");
     return 0;
 }

@@ -218,3 +218,27 @@ def test_tomopel_option_runs_the_models_and_leaves_the_default_alone():
     assert {"attention", "recurrence", "gated recurrence", "experts up"} <= set(line["tomopel"]["stages"]["prefill_512"])
     assert line["value"] == line["tomopel"]["decode_b8"]["tok_s"]
     assert line["prefill_kernels"]["tomopel_recurrence"]["ms"] > 0 and line["decode_kernels"]["tomopel_attention"]["ms"] > 0
+
+
+def test_pusazen_option_runs_the_models_and_leaves_the_default_alone():
+    """``--pusazen`` runs a Pusazen model beside the closest Tomopel, Rusolorn and Metitar models and prints one JSON line;
+    the sizes' config.json dicts are what the registry takes."""
+    import bench
+    from somi_inference_amd.config import config_from_dict
+    for sizes in bench.PUSAZEN_SIZES:
+        arch, config = config_from_dict(bench.pusazen_config_dict(sizes))
+        assert arch.name == "Pusazen" and [layer.type for layer in config.layers].count("mlstm") == bench.PUSAZEN_LAYERS["mlstm"]
+        assert len(config.layers) == sum(bench.PUSAZEN_LAYERS.values())
+        memory, right = config.layers[0].mixer, config_from_dict(bench.tomopel_config_dict(sizes))[1].layers[0].mixer.right
+        assert memory.heads * memory.dim * memory.vdim == right.heads * right.vdim * right.state
+        arch, dense = config_from_dict(bench.pusazen_closest_dense_config_dict(sizes))
+        assert arch.name == "Metitar" and dense.width == config.width and dense.layers[0].mlp.ff == config.layers[0].mlp.ff
+    done = subprocess.run([sys.executable, os.path.join(ROOT, "bench.py"), "--pusazen", "1b", "--steps", "16", "--warmup", "2",
+                           "--prefill-tokens", "512", "--context", "1024"], capture_output=True, text=True, timeout=900, cwd=ROOT)
+    assert done.returncode == 0, done.stderr[-3000:]
+    line = json.loads([row for row in done.stdout.splitlines() if row.startswith("{")][-1])
+    for model in ("pusazen", "closest", "closest_experts", "closest_dense"):
+        assert line[model]["decode_b8"]["tok_s"] > 0 and line[model]["prefill"]["512"]["value"] > 0
+    assert {"attention", "recurrence", "gates", "sum, norm", "experts gate_up"} <= set(line["pusazen"]["stages"]["prefill_512"])
+    assert line["value"] == line["pusazen"]["decode_b8"]["tok_s"]
+    assert line["prefill_kernels"]["pusazen_recurrence"]["ms"] > 0 and line["decode_kernels"]["pusazen_attention"]["ms"] > 0
